@@ -165,7 +165,9 @@ class SharedExpertSpec(BaseModel):
 
 class RoutedExpertsSpec(BaseModel):
     """Mixture of silu-GLU experts behind a router. ``score`` turns the router
-    logits into scores: softmax over all outputs, or sigmoid of each. The last
+    logits into scores: softmax over all outputs, sigmoid of each, or
+    ("top_softmax") the choice by the logits themselves and the softmax over
+    the chosen ones. The last
     ``identity`` router outputs are experts that return their input. The
     choice is made on score (+ correction, if the checkpoint has one) among
     the experts of the best ``group_keep`` of ``group_count`` groups of
@@ -180,14 +182,15 @@ class RoutedExpertsSpec(BaseModel):
     group_count: int = 1
     group_keep: int = 1
     ff: int
-    score: Literal["softmax", "sigmoid"] = "softmax"
+    score: Literal["softmax", "sigmoid", "top_softmax"] = "softmax"
     renormalize: bool = True
     correction: bool = True
     weight_on: Literal["output", "input"] = "output"
     shared: Optional[SharedExpertSpec] = None
     # the experts' form: silu(gate) * up, or the clamped GLU
-    # min(gate, limit) sigmoid(alpha min(gate, limit)) (clamp(up, +-limit) + 1)
-    act: Literal["silu", "clamped"] = "silu"
+    # min(gate, limit) sigmoid(alpha min(gate, limit)) (clamp(up, +-limit) + 1), or
+    # relu2, two-matrix experts W_down relu(W_up h)^2 without a gate matrix
+    act: Literal["silu", "clamped", "relu2"] = "silu"
     limit: float = 0.0
     alpha: float = 1.702
 
@@ -202,6 +205,25 @@ class LoopSpec(BaseModel):
     start: int
     stop: int
     times: int
+
+
+def loop_order(n: int, loop: Optional[LoopSpec]) -> List[tuple]:
+    """(layer index, starts a pass of the loop) per layer run of an n-layer
+    model, in execution order: the looped range runs ``times`` times in a row."""
+    if loop is None:
+        return [(i, False) for i in range(n)]
+    a, b = loop.start, loop.stop
+    return ([(i, False) for i in range(a)] + [(i, i == a) for i in range(a, b)] * loop.times +
+            [(i, False) for i in range(b, n)])
+
+
+def read_loop(lp: Optional[dict], n: int) -> Optional[LoopSpec]:
+    """The ``loop`` entry of a config.json whose model lists n layers."""
+    if not lp:
+        return None
+    if lp["times"] < 1 or not 0 <= lp["start"] < lp["stop"] <= n:
+        raise ValueError(f"loop {lp} does not fit {n} layers")
+    return LoopSpec(**lp)
 
 
 class MedilixLayerSpec(BaseModel):
@@ -236,14 +258,7 @@ class MedilixArchConfig(BaseModel):
         return len(self.layers)
 
     def layer_runs(self) -> List[tuple]:
-        """(layer index, starts a pass of the loop) per layer run, in
-        execution order: the looped range runs ``times`` times in a row."""
-        n = len(self.layers)
-        if self.loop is None:
-            return [(i, False) for i in range(n)]
-        a, b, times = self.loop.start, self.loop.stop, self.loop.times
-        looped = [(i, i == a) for i in range(a, b)] * times
-        return [(i, False) for i in range(a)] + looped + [(i, False) for i in range(b, n)]
+        return loop_order(len(self.layers), self.loop)
 
     @classmethod
     def from_checkpoint_config(cls, d: dict, shapes: Optional[dict] = None) -> "MedilixArchConfig":
@@ -285,13 +300,10 @@ class MedilixArchConfig(BaseModel):
                 raise ValueError(f"unknown layer type {kind!r}")
         emb = d.get("embedding") or {}
         bg = emb.get("bigram")
-        lp = d.get("loop")
-        if lp and (lp["times"] < 1 or not 0 <= lp["start"] < lp["stop"] <= len(layers)):
-            raise ValueError(f"loop {lp} does not fit {len(layers)} layers")
         return cls(vocab_size=d["vocab"], hidden_size=d["width"], rms_norm_eps=d["norm"]["eps"],
                    norm_groups=d["norm"].get("groups", 1), embed_scale=emb.get("scale", 1.0),
                    bigram=BigramSpec(**bg) if bg else None, layers=layers,
-                   loop=LoopSpec(**lp) if lp else None)
+                   loop=read_loop(d.get("loop"), len(layers)))
 
 
 def _medilix_preset(vocab, width, depth, heads, kv_heads, dim, mask, keep, r_heads, r_dim, m_heads, m_dim,
@@ -328,7 +340,10 @@ class LatentAttnSpec(BaseModel):
     ``rot_dim`` rotated entries; the token's down-projection gives the latent
     (``kv_rank`` entries, RMS-normed) and one rotated key part shared by all
     heads. Only those two are cached. Causal sliding window of ``mask_size``
-    positions (0 = plain causal); per-head sigmoid output gate."""
+    positions (0 = plain causal). Output gate: sigmoid of one logit per head
+    (``head_gate``), of one per output element (``elem_gate``: multiplies the
+    concatenated heads), or none. ``sink``: a learned number per head whose
+    exponential joins the softmax denominator without a value."""
 
     heads: int
     dim: int
@@ -339,14 +354,18 @@ class LatentAttnSpec(BaseModel):
     mask_size: int = 0
     rot: RotarySpec = Field(default_factory=RotarySpec)
     head_gate: bool = True
+    elem_gate: bool = False
+    sink: bool = False
 
 
 class ActFFSpec(BaseModel):
-    """Two-matrix feed-forward W_down act(W_up h); act = tanh-form gelu."""
+    """Feed-forward W_down act(W_up h), or W_down (act(W_gate h) * (W_up h)) if
+    ``gated``; act = tanh-form gelu."""
 
     kind: Literal["dense"] = "dense"
     ff: int
     act: Literal["gelu_tanh"] = "gelu_tanh"
+    gated: bool = False
 
 
 class MitunexLayerSpec(BaseModel):
@@ -607,6 +626,120 @@ def _pironex_preset(vocab, width, depth, heads, kv_heads, dim, mask, pool, m_hea
     return PironexArchConfig(vocab_size=vocab, hidden_size=width, embed_scale=1.0, canon_taps=taps, layers=layers)
 
 
+class RetentionSpec(BaseModel):
+    """Linear attention with one constant decay per head and rotary positions
+    on q and k: S <- decay_h S + k v^T, o = S^T q, k scaled by dim^-1/2 after
+    the rotation. Every head's o is RMS-normed without a weight and the
+    concatenation gated by silu(W_g h)."""
+
+    heads: int
+    dim: int
+    vdim: int
+    decay: List[float]
+    rot: RotarySpec = Field(default_factory=lambda: RotarySpec(layout="half"))
+
+
+class BavesunLayerSpec(BaseModel):
+    type: Literal["retention", "latent_attention"]
+    retention: Optional[RetentionSpec] = None
+    latent: Optional[LatentAttnSpec] = None
+    mlp: Optional[Union[ActFFSpec, RoutedExpertsSpec]] = None
+
+
+class BavesunArchConfig(BaseModel):
+    """A decoder of parallel layers with one norm, x <- x + (mixer(h) + ff(h)),
+    h = rms(x) (1 + w), each followed by a gated per-token side input
+    x <- x + rms(W_proj (gelu(W_gate x) * e)) w, e = the layer's part of the
+    token's row in a side table. Mixers: retention, or latent attention with a
+    sink and an elementwise gate; feed-forward: gated gelu, routed squared-relu
+    experts, or none. A range of layers may repeat with the same weights, every
+    pass with its own cache and state. The LM head is the embedding table
+    without its scale. Every size comes from the checkpoint's config.json."""
+
+    arch: Literal["bavesun"] = "bavesun"
+    vocab_size: int
+    hidden_size: int
+    rms_norm_eps: float = 1e-5
+    embed_scale: float = 1.0
+    side_dim: int = 0                   # 0 = no side input
+    layers: List[BavesunLayerSpec]
+    loop: Optional[LoopSpec] = None
+    max_position_embeddings: int = 1 << 24
+    tie_word_embeddings: bool = True
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    def layer_runs(self) -> List[int]:
+        """Layer index per layer run, in execution order."""
+        return [i for i, _ in loop_order(len(self.layers), self.loop)]
+
+    @classmethod
+    def from_checkpoint_config(cls, d: dict, shapes: Optional[dict] = None) -> "BavesunArchConfig":
+        """Parse the family's config.json (keys: vocab, width, norm.eps,
+        embedding.scale, token_side.dim, loop, layers[].type / .mixer / .mlp)."""
+        layers = []
+        for li, spec in enumerate(d["layers"]):
+            m, mlp, kind = spec["mixer"], spec.get("mlp"), spec["type"]
+            ff = None
+            if mlp:
+                if mlp["kind"] == "dense":
+                    ff = ActFFSpec(ff=mlp["ff"], gated=True)
+                elif mlp["kind"] == "moe":
+                    r = mlp["router"]
+                    ff = RoutedExpertsSpec(experts=r["experts"], top=r["top"], ff=mlp["expert"]["ff"],
+                                           score="top_softmax", correction=False, act="relu2")
+                else:
+                    raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+            rot = m.get("rot") or {}
+            if kind == "retention":
+                if len(m["decay"]) != m["heads"]:
+                    raise ValueError(f"layer {li}: {len(m['decay'])} decays for {m['heads']} heads")
+                layers.append(BavesunLayerSpec(type=kind, mlp=ff, retention=RetentionSpec(
+                    heads=m["heads"], dim=m["dim"], vdim=m["vdim"], decay=list(m["decay"]),
+                    rot=RotarySpec(base=rot.get("base", 10000.0), dims=rot.get("dims") or 0, layout="half"))))
+            elif kind == "latent_attention":
+                if rot.get("dims", m["rot_dim"]) != m["rot_dim"]:
+                    raise ValueError("the rotated part of a latent-attention head is rotated whole")
+                layers.append(BavesunLayerSpec(type=kind, mlp=ff, latent=LatentAttnSpec(
+                    heads=m["heads"], dim=m["dim"], rot_dim=m["rot_dim"], vdim=m["vdim"], kv_rank=m["kv_rank"],
+                    scale=m["scale"], rot=RotarySpec(base=rot.get("base", 10000.0), dims=m["rot_dim"]),
+                    head_gate=False, elem_gate=True, sink=True)))
+            else:
+                raise ValueError(f"unknown layer type {kind!r}")
+        return cls(vocab_size=d["vocab"], hidden_size=d["width"], rms_norm_eps=d["norm"]["eps"],
+                   embed_scale=(d.get("embedding") or {}).get("scale", 1.0),
+                   side_dim=(d.get("token_side") or {}).get("dim") or 0, layers=layers,
+                   loop=read_loop(d.get("loop"), len(layers)))
+
+
+def _bavesun_preset(vocab, width, depth, r_heads, r_dim, r_vdim, heads, dim, rot_dim, vdim, kv_rank, ff, experts,
+                    top, expert_ff, side_dim, pattern="RlrL", loop=None) -> BavesunArchConfig:
+    """Random-init presets of the family: ``pattern`` repeats over the depth
+    ('r' retention, 'l' latent attention; upper case: dense feed-forward,
+    lower case: routed experts)."""
+    import math as _math
+
+    layers = []
+    for i in range(depth):
+        c = pattern[i % len(pattern)]
+        mlp = (ActFFSpec(ff=ff, gated=True) if c.isupper() else
+               RoutedExpertsSpec(experts=experts, top=top, ff=expert_ff, score="top_softmax", correction=False,
+                                 act="relu2"))
+        if c in "rR":
+            layers.append(BavesunLayerSpec(type="retention", mlp=mlp, retention=RetentionSpec(
+                heads=r_heads, dim=r_dim, vdim=r_vdim, decay=[1.0 - 2.0 ** (-5 - 6.0 * h / r_heads) for h in range(r_heads)],
+                rot=RotarySpec(base=10000.0, dims=r_dim, layout="half"))))
+        else:
+            layers.append(BavesunLayerSpec(type="latent_attention", mlp=mlp, latent=LatentAttnSpec(
+                heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, kv_rank=kv_rank,
+                scale=1.0 / _math.sqrt(dim + rot_dim), rot=RotarySpec(base=1e6, dims=rot_dim),
+                head_gate=False, elem_gate=True, sink=True)))
+    return BavesunArchConfig(vocab_size=vocab, hidden_size=width, embed_scale=_math.sqrt(width), side_dim=side_dim,
+                             layers=layers, loop=LoopSpec(**loop) if loop else None)
+
+
 class HybridLayerSpec(BaseModel):
     type: Literal["parallel", "channel_delta"]
     parallel: Optional[ParallelMixerSpec] = None
@@ -837,6 +970,23 @@ MODEL_PRESETS: dict = {
         vocab=32000, width=2048, depth=6, heads=16, kv_heads=4, dim=128, mask=1024, pool=64, m_heads=32,
         m_vdim=64, m_state=128, m_groups=4, l_heads=16, l_dim=128, l_rot=64, l_vdim=128, l_rank=512, l_mask=1024,
         experts=8, top=2, expert_ff=4096, shared_ff=1024),
+    # Bavesun family (parallel layers with one norm; retention and latent
+    # attention with a sink; gated gelu and squared-relu experts; a per-layer
+    # token side input; looped layer range)
+    "tiny-bavesun": _bavesun_preset(
+        vocab=512, width=64, depth=4, r_heads=4, r_dim=16, r_vdim=24, heads=4, dim=16, rot_dim=8, vdim=24,
+        kv_rank=32, ff=96, experts=6, top=2, expert_ff=48, side_dim=8, loop={"start": 1, "stop": 3, "times": 2}),
+    "mid-bavesun": _bavesun_preset(
+        vocab=2048, width=512, depth=4, r_heads=8, r_dim=64, r_vdim=128, heads=8, dim=64, rot_dim=32, vdim=64,
+        kv_rank=128, ff=1024, experts=8, top=2, expert_ff=512, side_dim=32),
+    # layer shapes of real models at reduced depth, beside llama-/mitunex-{1b,8b}-l6
+    # (a two-matrix expert of ff 3/2 f has as many weights as a three-matrix one of f)
+    "bavesun-8b-l6": _bavesun_preset(
+        vocab=32000, width=4096, depth=6, r_heads=32, r_dim=128, r_vdim=128, heads=32, dim=128, rot_dim=64,
+        vdim=128, kv_rank=512, ff=14336, experts=8, top=2, expert_ff=10752, side_dim=256, pattern="Rl"),
+    "bavesun-1b-l6": _bavesun_preset(
+        vocab=32000, width=2048, depth=6, r_heads=16, r_dim=64, r_vdim=128, heads=16, dim=128, rot_dim=64,
+        vdim=128, kv_rank=512, ff=8192, experts=8, top=2, expert_ff=6144, side_dim=128, pattern="Rl"),
 }
 
 
@@ -939,11 +1089,12 @@ class EngineConfig(BaseModel):
         with open(cfg_path) as f:
             hf = json.load(f)
         family = str(hf.get("architecture", "")).lower()
-        if family in ("zutalix", "medilix", "mitunex", "pironex"):
+        if family in ("zutalix", "medilix", "mitunex", "pironex", "bavesun"):
             from .weights import safetensors_shapes
 
             reader = {"zutalix": HybridArchConfig, "medilix": MedilixArchConfig,
-                      "mitunex": MitunexArchConfig, "pironex": PironexArchConfig}[family]
+                      "mitunex": MitunexArchConfig, "pironex": PironexArchConfig,
+                      "bavesun": BavesunArchConfig}[family]
             return reader.from_checkpoint_config(hf, safetensors_shapes(os.path.dirname(cfg_path)))
         arch = "mixtral" if "mixtral" in hf.get("model_type", "").lower() or hf.get("num_local_experts") else "llama"
         return ModelArchConfig(

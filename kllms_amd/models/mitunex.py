@@ -92,15 +92,16 @@ class MitunexForCausalLM(ListedLayerLM):
             g = torch.Generator(device="cpu")
             g.manual_seed(int(hashlib.md5(f"{seed}/{name}".encode()).hexdigest()[:15], 16))
             leaf = name.split(".")[-1]
-            if leaf in ("norm", "norm1", "norm2"):
-                t = torch.ones(dst.shape)
-            elif leaf == "embed":
-                t = torch.randn(dst.shape, generator=g)
-            elif leaf == "pos":
-                t = torch.randn(dst.shape, generator=g) * 0.3
-            else:
-                t = torch.randn(dst.shape, generator=g) / math.sqrt(dst.shape[-1])
-            dst.copy_(t.to(device=dst.device, dtype=dst.dtype))
+            for part in dst if isinstance(dst, (list, tuple)) else [dst]:
+                if leaf in ("norm", "norm1", "norm2"):
+                    t = torch.ones(part.shape)
+                elif leaf == "embed":
+                    t = torch.randn(part.shape, generator=g)
+                elif leaf == "pos":
+                    t = torch.randn(part.shape, generator=g) * 0.3
+                else:
+                    t = torch.randn(part.shape, generator=g) / math.sqrt(part.shape[-1])
+                part.copy_(t.to(device=part.device, dtype=part.dtype))
 
     # --- forward ------------------------------------------------------------------
     def forward_hidden(self, input_ids: torch.Tensor, batch: ForwardBatch) -> torch.Tensor:

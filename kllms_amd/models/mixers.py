@@ -3,7 +3,8 @@ parameters: block-local softmax attention over the paged cache, decayed
 linear attention, the gated delta rule with per-channel decay and short
 convolutions, the clamped GLU; windowed attention with kept first tokens and
 a sink, the wkv and mlstm recurrences, routed experts; latent attention and
-the two-matrix gelu feed-forward. Each runs on "segment" batches
+the gelu feed-forwards; retention, the zero-centred norm weight and the token
+side input. Each runs on "segment" batches
 (ForwardBatch.seg_start / state_slots / token_seg): any mix of prompt
 portions and single decoded tokens, attention keys found through the block
 table and recurrent state carried in per-sequence slots.
@@ -26,7 +27,7 @@ import torch.nn.functional as F
 from .. import ops
 from ..engine.config import (ActFFSpec, BlockAttnSpec, ChannelDeltaSpec, DecayLinearAttnSpec, GluSpec,
                              LatentAttnSpec, Mamba2Spec, MaskedAttnSpec, MlstmSpec, ParallelMixerSpec,
-                             PoolWindowAttnSpec, RotarySpec, RoutedExpertsSpec, WkvSpec)
+                             PoolWindowAttnSpec, RetentionSpec, RotarySpec, RoutedExpertsSpec, WkvSpec)
 from ..engine.kvcache import LayerCacheSpec, LayerState
 
 
@@ -394,8 +395,11 @@ class LatentAttention(nn.Module):
     and the attention proper runs in the latent space for all heads against
     the same cached rows: W_uk is applied to the queries before it (one
     batched product over the heads) and W_uv to its result. Sliding causal
-    window, per-head sigmoid output gate; q, the down-projection and the gate
-    share one input GEMM."""
+    window or plain causal, optional sink (a learned number per head in the
+    softmax denominator), sigmoid output gate per head, per element of the
+    concatenated heads, or none; q, the down-projection and the gate share one
+    input GEMM. Both batched products take a right operand stored row by row
+    in the layout they read (W_uv per head as [C, V])."""
 
     def __init__(self, spec: LatentAttnSpec, hidden: int, eps: float, dtype):
         super().__init__()
@@ -404,12 +408,14 @@ class LatentAttention(nn.Module):
         self.eps = eps
         H, D, R, V, C = spec.heads, spec.dim, spec.rot_dim, spec.vdim, spec.kv_rank
         parts = [("q", H * (D + R)), ("dkv", C + R)]
-        if spec.head_gate:
-            parts.append(("g", H))
+        assert not (spec.head_gate and spec.elem_gate)
+        if spec.head_gate or spec.elem_gate:
+            parts.append(("g", H if spec.head_gate else H * V))
         self.inp = FusedInput(hidden, parts, dtype)
         self.dkv_norm = _param(C, dtype=torch.float32)
         self.uk = _param(H, D, C, dtype=dtype)
-        self.uv = _param(H, V, C, dtype=dtype)
+        self.uv = _param(H, C, V, dtype=dtype)
+        self.sink = _param(H, dtype=torch.float32) if spec.sink else None
         self.o_proj = _param(hidden, H * V, dtype=dtype)
         self.register_buffer("inv_freq", rotary_inv_freq(spec.rot), persistent=False)
 
@@ -433,18 +439,98 @@ class LatentAttention(nn.Module):
         lat = ops.attn_latent_paged(q_abs.transpose(0, 1), q, st.k, batch.block_tables, batch.token_seg,
                                     batch.positions, sp.scale, sp.mask_size,
                                     s(y, "g") if sp.head_gate else None, D,
-                                    tile_rows=1 if single else 0)                 # [T, H, C]
+                                    tile_rows=1 if single else 0, sink=self.sink)  # [T, H, C]
         att = torch.empty((T, H * V), dtype=y.dtype, device=y.device)
-        torch.bmm(lat.transpose(0, 1), self.uv.transpose(1, 2), out=att.view(T, H, V).transpose(0, 1))
+        torch.bmm(lat.transpose(0, 1), self.uv, out=att.view(T, H, V).transpose(0, 1))
+        if sp.elem_gate:
+            ops.sigmoid_gate_(att, s(y, "g"))
         return F.linear(att, self.o_proj)
 
     def checkpoint_map(self, pre: str) -> Dict[str, torch.Tensor]:
         m = {pre + n: self.inp.slot(n) for n in self.inp.parts}
         m[pre + "dkv.norm"] = self.dkv_norm
         m[pre + "uk"] = self.uk.view(-1, self.spec.kv_rank)
-        m[pre + "uv"] = self.uv.view(-1, self.spec.kv_rank)
+        m[pre + "uv"] = [head.t() for head in self.uv]      # the checkpoint's rows, V per head
+        if self.sink is not None:
+            m[pre + "sink"] = self.sink
         m[pre + "o"] = self.o_proj
         return m
+
+
+class Retention(nn.Module):
+    """S <- decay_h S + k v^T, o = S^T q with one constant decay per head; q
+    and k are rotated (entry i with i + dims/2), k then scaled by dim^-1/2.
+    Every head's o is RMS-normed (no weight), the concatenation times
+    silu(W_g h) is projected. From the projections to the read-out everything
+    is fp32. State: S [H, D, V] fp32. q, k, v and the gate share one input
+    GEMM."""
+
+    def __init__(self, spec: RetentionSpec, hidden: int, eps: float, dtype):
+        super().__init__()
+        assert len(spec.decay) == spec.heads and spec.rot.layout == "half" and not spec.rot.scaling
+        assert spec.rot.dims % 2 == 0 and spec.rot.dims <= spec.dim
+        self.spec = spec
+        self.eps = eps
+        hd, hv = spec.heads * spec.dim, spec.heads * spec.vdim
+        self.inp = FusedInput(hidden, [("q", hd), ("k", hd), ("v", hv), ("g", hv)], dtype)
+        self.o_proj = _param(hidden, hv, dtype=dtype)
+        self.register_buffer("inv_freq", rotary_inv_freq(spec.rot), persistent=False)
+        self.register_buffer("decay", torch.tensor(spec.decay, dtype=torch.float64).to(torch.float32),
+                             persistent=False)
+
+    def cache_spec(self) -> LayerCacheSpec:
+        sp = self.spec
+        return LayerCacheSpec(rec=(sp.heads, sp.dim, sp.vdim))
+
+    def forward(self, h: torch.Tensor, batch, st: LayerState) -> torch.Tensor:
+        sp = self.spec
+        y = self.inp(h)
+        s = self.inp.split
+        o = ops.retention(s(y, "q").unflatten(1, (sp.heads, sp.dim)), s(y, "k").unflatten(1, (sp.heads, sp.dim)),
+                          s(y, "v").unflatten(1, (sp.heads, sp.vdim)), self.decay, batch.positions, self.inv_freq,
+                          st.rec, batch.state_slots, batch.cu_seqlens, batch.seg_start)
+        r = ops.gated_rmsnorm(o, None, s(y, "g"), self.eps, self.o_proj.dtype, "silu")
+        return F.linear(r, self.o_proj)
+
+    def checkpoint_map(self, pre: str) -> Dict[str, torch.Tensor]:
+        m = {pre + n: self.inp.slot(n) for n in self.inp.parts}
+        m[pre + "o"] = self.o_proj
+        return m
+
+
+class CentredNormWeight(nn.Module):
+    """Weight of a norm that is stored as its distance from one: ``scale``
+    (fp32, what the norm kernels multiply with) is 1 + weight, formed by
+    ``fold()`` once the weight is in place."""
+
+    def __init__(self, width: int):
+        super().__init__()
+        self.weight = _param(width, dtype=torch.float32)
+        self.register_buffer("scale", torch.ones(width, dtype=torch.float32), persistent=False)
+
+    def fold(self) -> None:
+        self.scale.copy_(1.0 + self.weight)
+
+
+class TokenSide(nn.Module):
+    """A layer's per-token side input: with e the layer's columns of the
+    token's row in a side table shared by the layers,
+    y = W_proj (gelu(W_gate x) * e); the caller adds rms(y) * norm to the
+    stream."""
+
+    def __init__(self, hidden: int, dim: int, index: int, dtype):
+        super().__init__()
+        self.col0, self.dim = index * dim, dim
+        self.gate = _param(dim, hidden, dtype=dtype)
+        self.proj = _param(hidden, dim, dtype=dtype)
+        self.norm = _param(hidden, dtype=torch.float32)
+
+    def forward(self, x: torch.Tensor, input_ids: torch.Tensor, table: torch.Tensor) -> torch.Tensor:
+        g = ops.gelu_mul_rows(F.linear(x, self.gate), table, input_ids, self.col0)
+        return F.linear(g, self.proj)
+
+    def checkpoint_map(self, pre: str) -> Dict[str, torch.Tensor]:
+        return {pre + "gate": self.gate, pre + "proj": self.proj, pre + "norm": self.norm}
 
 
 class PoolWindowAttention(nn.Module):
@@ -583,18 +669,25 @@ class Mamba2Mixer(nn.Module):
 
 
 class ActFF(nn.Module):
-    """y = W_down act(W_up h) with the tanh-form gelu."""
+    """y = W_down act(W_up h), or W_down (act(W_gate h) * (W_up h)) when gated
+    (gate and up share one GEMM), with the tanh-form gelu."""
 
     def __init__(self, spec: ActFFSpec, hidden: int, dtype):
         super().__init__()
         self.spec = spec
-        self.up = _param(spec.ff, hidden, dtype=dtype)
+        self.inp = FusedInput(hidden, [("gate", spec.ff), ("up", spec.ff)], dtype) if spec.gated else None
+        self.up = None if spec.gated else _param(spec.ff, hidden, dtype=dtype)
         self.down = _param(hidden, spec.ff, dtype=dtype)
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
+        if self.inp is not None:
+            y = self.inp(h)
+            return F.linear(ops.gelu_glu(self.inp.split(y, "gate"), self.inp.split(y, "up")), self.down)
         return F.linear(ops.gelu_tanh(F.linear(h, self.up)), self.down)
 
     def checkpoint_map(self, pre: str) -> Dict[str, torch.Tensor]:
+        if self.inp is not None:
+            return {pre + "gate": self.inp.slot("gate"), pre + "up": self.inp.slot("up"), pre + "down": self.down}
         return {pre + "up": self.up, pre + "down": self.down}
 
 
@@ -620,7 +713,7 @@ class WkvMixer(nn.Module):
         self.hidden = hidden
         hd = spec.heads * spec.dim
         self.mu = _param(len(self.STREAMS), hidden, dtype=torch.float32)
-        self.rkvg = _param(4, hd, hidden, dtype=dtype)            # one batched GEMM for r, k, v, g
+        self.rkvg = _param(4, hidden, hd, dtype=dtype)   # r, k, v, g as right operands [in, out] of one batched GEMM
         self.w1 = _param(spec.decay_rank, hidden, dtype=torch.float32)
         self.w2 = _param(hd, spec.decay_rank, dtype=torch.float32)
         self.w0 = _param(hd, dtype=torch.float32)
@@ -637,9 +730,9 @@ class WkvMixer(nn.Module):
         mixes, mix_w = ops.token_shift_mix(h, self.mu, st.shift, batch.state_slots, batch.cu_seqlens,
                                            batch.seg_start, batch.token_seg, 4)
         if h.shape[0] <= self.BATCHED_MAX_ROWS:
-            y = torch.bmm(mixes, self.rkvg.transpose(1, 2))                   # [4, T, H*D], one launch
+            y = torch.bmm(mixes, self.rkvg)                                   # [4, T, H*D], one launch
         else:
-            y = [F.linear(mixes[i], self.rkvg[i]) for i in range(4)]
+            y = [torch.mm(mixes[i], self.rkvg[i]) for i in range(4)]
         d = F.linear(torch.tanh(F.linear(mix_w[0], self.w1)), self.w2)       # fp32 [T, H*D]
         hd = (sp.heads, sp.dim)
         o = ops.wkv_recurrence(y[0].unflatten(1, hd), y[1].unflatten(1, hd), y[2].unflatten(1, hd), d,
@@ -650,7 +743,7 @@ class WkvMixer(nn.Module):
     def checkpoint_map(self, pre: str) -> Dict[str, torch.Tensor]:
         m = {pre + "mu." + n: self.mu[i] for i, n in enumerate(self.STREAMS)}
         for i, n in enumerate(self.STREAMS[:4]):
-            m[pre + n] = self.rkvg[i]
+            m[pre + n] = self.rkvg[i].t()
         for n in ("w1", "w2", "w0", "u", "norm"):
             m[pre + n] = getattr(self, n)
         m[pre + "o"] = self.o_proj
@@ -707,9 +800,10 @@ class MlstmMixer(nn.Module):
 
 class RoutedExperts(nn.Module):
     """Mixture of GLU experts (silu(gate) * up, or the clamped form with
-    limits of their own for the routed and the shared expert). The router runs in fp32: scores are the
-    softmax over all outputs or the sigmoid of each; the choice is made on
-    score (+ correction) within the best groups of neighbouring experts; the
+    limits of their own for the routed and the shared expert) or of two-matrix
+    squared-relu experts. The router runs in fp32: scores are the softmax over
+    all outputs, the sigmoid of each, or the softmax over the chosen logits;
+    the choice is made on score (+ correction) within the best groups of neighbouring experts; the
     chosen scores, renormalised or as they are, weigh the experts — their
     outputs, or (``weight_on = "input"``) their inputs: expert(w h). The last
     ``identity`` router outputs stand for experts that return their input and
@@ -741,8 +835,12 @@ class RoutedExperts(nn.Module):
         assert not (spec.weight_on == "input" and spec.identity), "identity experts take their weight on the output"
         self.router = _param(n, hidden, dtype=torch.float32)
         self.correction = _param(n, dtype=torch.float32) if spec.correction else None
-        self.w_gate_up = _param(spec.experts, 2 * spec.ff, hidden, dtype=dtype)
-        self.w_down = _param(spec.experts, hidden, spec.ff, dtype=dtype)
+        # [in, out] per expert: right operands of plain and batched products as they lie in memory.
+        # Columns of w_in: gate | up, or up alone
+        self.glu = spec.act != "relu2"
+        self.w_in = _param(spec.experts, hidden, (2 if self.glu else 1) * spec.ff, dtype=dtype)
+        self.w_down = _param(spec.experts, spec.ff, hidden, dtype=dtype)
+        assert self.glu or spec.shared is None, "the shared expert has the GLU form"
         self.shared_inp = self.shared_down = None
         if spec.shared is not None:
             sff = spec.shared.ff
@@ -754,6 +852,12 @@ class RoutedExperts(nn.Module):
         if sp.act == "clamped":
             return ops.gated_act(gate, up, sp.limit if limit is None else limit, sp.alpha, 1.0)
         return ops.silu_glu(gate, up)
+
+    def _act_rows(self, y: torch.Tensor) -> torch.Tensor:
+        """[n, gate | up] (or [n, up]) input products of routed experts -> [n, ff]."""
+        if not self.glu:
+            return ops.relu2(y)
+        return self._act(y[:, :self.spec.ff], y[:, self.spec.ff:])
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         sp = self.spec
@@ -769,9 +873,8 @@ class RoutedExperts(nn.Module):
                 xin = ops.moe_spread_rows(h, idx, w, E)
             else:
                 xin = h.unsqueeze(0).expand(E, T, W)
-            gu = torch.bmm(xin, self.w_gate_up.transpose(1, 2)).view(E * T, 2 * sp.ff)
-            act = self._act(gu[:, :sp.ff], gu[:, sp.ff:]).view(E, T, sp.ff)
-            rows = torch.bmm(act, self.w_down.transpose(1, 2)).view(E * T, W)
+            act = self._act_rows(torch.bmm(xin, self.w_in).flatten(0, 1)).view(E, T, sp.ff)
+            rows = torch.bmm(act, self.w_down).view(E * T, W)
         else:
             flat = idx.reshape(-1).long().clamp(max=E)                # identity experts sort last
             order = torch.argsort(flat, stable=True)
@@ -785,8 +888,8 @@ class RoutedExperts(nn.Module):
             s0 = 0
             for e, c in enumerate(counts):
                 if c:
-                    gu = F.linear(xs[s0:s0 + c], self.w_gate_up[e])
-                    rows[s0:s0 + c] = F.linear(self._act(gu[:, :sp.ff], gu[:, sp.ff:]), self.w_down[e])
+                    act = self._act_rows(torch.mm(xs[s0:s0 + c], self.w_in[e]))
+                    torch.mm(act, self.w_down[e], out=rows[s0:s0 + c])
                     s0 += c
             pos = torch.empty(T * top, dtype=torch.int32, device=h.device)
             pos[order] = torch.arange(T * top, dtype=torch.int32, device=h.device)
@@ -805,9 +908,10 @@ class RoutedExperts(nn.Module):
         if self.correction is not None:
             m[pre + "correction"] = self.correction
         for e in range(self.spec.experts):
-            m[f"{pre}e{e}.gate"] = self.w_gate_up[e, :ff]
-            m[f"{pre}e{e}.up"] = self.w_gate_up[e, ff:]
-            m[f"{pre}e{e}.down"] = self.w_down[e]
+            if self.glu:
+                m[f"{pre}e{e}.gate"] = self.w_in[e, :, :ff].t()
+            m[f"{pre}e{e}.up"] = self.w_in[e, :, -ff:].t()
+            m[f"{pre}e{e}.down"] = self.w_down[e].t()
         if self.shared_inp is not None:
             for n in ("gate", "up", "sg"):
                 m[f"{pre}shared.{n}"] = self.shared_inp.slot(n)

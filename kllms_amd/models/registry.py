@@ -30,7 +30,11 @@ def model_class(arch: str):
         from .pironex import PironexForCausalLM
 
         return PironexForCausalLM
+    if arch == "bavesun":
+        from .bavesun import BavesunForCausalLM
+
+        return BavesunForCausalLM
     raise ValueError(f"no model registered for architecture {arch!r}")
 
 
-ARCHITECTURES = ("llama", "mixtral", "zutalix", "medilix", "mitunex", "pironex")
+ARCHITECTURES = ("llama", "mixtral", "zutalix", "medilix", "mitunex", "pironex", "bavesun")

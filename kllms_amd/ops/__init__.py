@@ -363,12 +363,15 @@ def linear_attn_decay(q, k, v, decay, state, state_slots, cu_seqlens, seg_start)
     return torch_ref.linear_attn_decay(q, k, v, decay, state, state_slots, cu_seqlens, seg_start)
 
 
-def gated_rmsnorm(o, weight, gate, eps, out_dtype):
+def gated_rmsnorm(o, weight, gate, eps, out_dtype, gate_act="sigmoid"):
+    """Grouped RMS norm of o [T, groups, S] fp32 (weight [S] or None) times
+    the activated gate (sigmoid or silu)."""
     if _gpu(o):
         out = torch.empty((o.shape[0], o.shape[1] * o.shape[2]), dtype=out_dtype, device=o.device)
-        _seq().gated_rmsnorm(out, o, weight, gate, eps, False)
+        _seq().gated_rmsnorm(out, o, weight if weight is not None else _none(o), gate, eps,
+                             0 if gate_act == "sigmoid" else 2)
         return out
-    return torch_ref.gated_rmsnorm(o, weight, gate, eps, out_dtype)
+    return torch_ref.gated_rmsnorm(o, weight, gate, eps, out_dtype, gate_act)
 
 
 def causal_conv_silu(x, w, conv_state, state_slots, cu_seqlens, seg_start, token_seg, bias=None):
@@ -510,10 +513,13 @@ def mlstm_mix_out(q, k, v, gates, gate_bias, cap, state, state_slots, cu_seqlens
 def head_rmsnorm_gate(o, weight, gate, eps, gate_act, out_dtype):
     if _gpu(o):
         out = torch.empty((o.shape[0], o.shape[1] * o.shape[2]), dtype=out_dtype, device=o.device)
-        _seq().head_rmsnorm_gate(out, o, weight, gate, eps, 0 if gate_act == "sigmoid" else 1,
-                                 _none(o, torch.float32))
+        _seq().head_rmsnorm_gate(out, o, weight, gate, eps,
+                                 0 if gate_act == "sigmoid" else 1, _none(o, torch.float32))
         return out
     return torch_ref.head_rmsnorm_gate(o, weight, gate, eps, gate_act, out_dtype)
+
+
+_SCORE_KINDS = {"softmax": 0, "sigmoid": 1, "top_softmax": 2}
 
 
 def moe_route(z, correction, top, group_count, group_keep, score="softmax", renormalize=True):
@@ -523,7 +529,7 @@ def moe_route(z, correction, top, group_count, group_keep, score="softmax", reno
         w = torch.empty((z.shape[0], top), dtype=torch.float32, device=z.device)
         _seq().moe_route(idx, w, _none(z, torch.int32), z, _none(z),
                          correction if correction is not None else _none(z), int(top), int(group_count),
-                         int(group_keep), 0, 0 if score == "softmax" else 1, bool(renormalize))
+                         int(group_keep), 0, _SCORE_KINDS[score], bool(renormalize))
         return idx, w
     return torch_ref.moe_route(z, correction, top, group_count, group_keep, score, renormalize)
 
@@ -541,7 +547,7 @@ def moe_route_rows(h, router, correction, top, group_count, group_keep, experts,
         _seq().moe_route(idx, w, rowidx if rowidx is not None else _none(h, torch.int32), h, router,
                          correction if correction is not None else _none(router),
                          int(top), int(group_count), int(group_keep), int(experts),
-                         0 if score == "softmax" else 1, bool(renormalize))
+                         _SCORE_KINDS[score], bool(renormalize))
         return idx, w, rowidx
     z = torch.nn.functional.linear(h.float(), router)
     idx, w = torch_ref.moe_route(z, correction, top, group_count, group_keep, score, renormalize)
@@ -614,10 +620,11 @@ def latent_kv_store(q, dkv, w_norm, eps, positions, inv_freq, cache, slot_mappin
 
 
 def attn_latent_paged(q_abs, q, cache, block_tables, token_seg, positions, scale, mask_size, gate, nope_dim,
-                      tile_rows: int = 0, use_mfma: bool = True, key_splits: int = 0):
+                      tile_rows: int = 0, use_mfma: bool = True, key_splits: int = 0, sink=None):
     """Sliding-window softmax attention over the paged latent cache in the
     absorbed form (one shared key/value row per token for all heads):
-    returns the heads' weighted latent sums [T, H, C], gated per head.
+    returns the heads' weighted latent sums [T, H, C], gated per head. sink
+    [H] fp32: one more term exp(sink_h) in the softmax denominator.
     GPU: bf16 rows go through the matrix-unit kernel when the sizes fit it
     (``tile_rows`` = query rows per workgroup, 0 = as many as fit 32 (row,
     head) columns; 1 suits steps of single decoded tokens), fp32 rows and
@@ -638,14 +645,24 @@ def attn_latent_paged(q_abs, q, cache, block_tables, token_seg, positions, scale
             ns = key_splits or max(1, min((tiles + 3) // 4, 512 // max(1, groups)))
             ns = max(1, min(ns, tiles, 64))
         f = torch.float32
-        part_o = torch.empty((T, H, ns, C), dtype=f, device=q.device) if ns > 1 else _none(q, f)
-        part_ml = torch.empty((T, H, ns, 2), dtype=f, device=q.device) if ns > 1 else _none(q, f)
+        f_none = _none(q, f)
+        part_o = torch.empty((T, H, ns, C), dtype=f, device=q.device) if ns > 1 else f_none
+        part_ml = torch.empty((T, H, ns, 2), dtype=f, device=q.device) if ns > 1 else f_none
         _seq().attn_latent_paged(out, q_abs, q, cache, block_tables, token_seg, positions,
                                  gate if gate is not None else _none(q), float(scale), int(mask_size),
-                                 int(nope_dim), int(tile_rows), bool(use_mfma), part_o, part_ml)
+                                 int(nope_dim), int(tile_rows), bool(use_mfma), part_o, part_ml,
+                                 sink if sink is not None else f_none)
         return out
     return torch_ref.attn_latent_paged(q_abs, q, cache, block_tables, token_seg, positions, scale, mask_size,
-                                       gate, nope_dim)
+                                       gate, nope_dim, sink)
+
+
+def sigmoid_gate_(x, gate) -> None:
+    """x [T, C] *= sigmoid(gate) element by element; gate a row view."""
+    if _gpu(x):
+        _seq().sigmoid_gate(x, gate)
+        return
+    torch_ref.sigmoid_gate_(x, gate)
 
 
 def attn_window_sink(q, st, batch, spec, gate):
@@ -759,6 +776,53 @@ def gate_group_rmsnorm(o, weight, gate, eps, out_dtype):
     """(o * silu(gate)) RMS-normed in groups, times weight: o [T, groups, S] fp32."""
     if _gpu(o):
         out = torch.empty((o.shape[0], o.shape[1] * o.shape[2]), dtype=out_dtype, device=o.device)
-        _seq().gated_rmsnorm(out, o, weight, gate, eps, True)
+        _seq().gated_rmsnorm(out, o, weight, gate, eps, 1)
         return out
     return torch_ref.gate_group_rmsnorm(o, weight, gate, eps, out_dtype)
+
+
+def retention(q, k, v, decay, positions, inv_freq, state, state_slots, cu_seqlens, seg_start):
+    """Half-split rotation of q and k, k scaled by D^-1/2, then
+    S <- decay_h S + k v^T, o = S^T q over segments; o [T, H, V] fp32."""
+    if _gpu(q):
+        o = torch.empty((q.shape[0], q.shape[1], v.shape[2]), dtype=torch.float32, device=q.device)
+        _seq().retention(o, q, k, v, decay, positions, inv_freq, state, state_slots, cu_seqlens, seg_start)
+        return o
+    return torch_ref.retention(q, k, v, decay, positions, inv_freq, state, state_slots, cu_seqlens, seg_start)
+
+
+def gelu_glu(gate, up):
+    """gelu(gate) * up (tanh form) of two row views, in gate's dtype."""
+    if _gpu(gate):
+        out = torch.empty(gate.shape, dtype=gate.dtype, device=gate.device)
+        _seq().gelu_glu(out, gate, up)
+        return out
+    return torch_ref.gelu_glu(gate, up)
+
+
+def relu2(x):
+    """max(x, 0)^2 of a [T, C] row view, in x's dtype."""
+    if _gpu(x):
+        out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+        _seq().relu2(out, x)
+        return out
+    return torch_ref.relu2(x)
+
+
+def gelu_mul_rows(z, table, ids, col0: int):
+    """gelu(z [T, C]) * table[ids, col0 : col0 + C] in z's dtype."""
+    if _gpu(z):
+        out = torch.empty(z.shape, dtype=z.dtype, device=z.device)
+        _seq().gelu_mul_rows(out, z, table, ids, int(col0))
+        return out
+    return torch_ref.gelu_mul_rows(z, table, ids, col0)
+
+
+def add_cast(x, a, b, out_dtype):
+    """x (fp32 residual, in place) += a + b (b may be None); returns x in
+    out_dtype (fp32: x itself)."""
+    if _gpu(x):
+        out = x if out_dtype == torch.float32 else torch.empty(x.shape, dtype=out_dtype, device=x.device)
+        _seq().add_cast(_none(x, out_dtype) if out is x else out, x, a, b if b is not None else _none(a))
+        return out
+    return torch_ref.add_cast(x, a, b, out_dtype)

@@ -18,7 +18,14 @@ void seq_launch_latent_kv_store(void*, const void*, const float*, float, const i
                                 const int64_t*, int, int, int, int, int, int, int, int, hipStream_t);
 void seq_launch_attn_latent_paged(void*, const void*, const void*, const void*, const int*, const int*,
                                   const int64_t*, const void*, float, int, int, int, int, int, int, int, int,
-                                  int64_t, int64_t, int, int, int, int, float*, float*, int, int, hipStream_t);
+                                  int64_t, int64_t, int, int, int, int, float*, float*, int, const float*, int,
+                                  hipStream_t);
+void seq_launch_act_pair(void*, const void*, const void*, const int64_t*, int64_t, int, int, int, int64_t, int, int,
+                         hipStream_t);
+void seq_launch_add_cast(void*, float*, const void*, const void*, int64_t, int, hipStream_t);
+void seq_launch_retention(float*, const void*, const void*, const void*, const float*, const int64_t*, const float*,
+                          float*, float*, const int*, const int*, const int*, int, int, int, int, int, int, int, int,
+                          int, int, hipStream_t);
 void seq_launch_rmsnorm_cast(void*, const float*, const float*, int, int, float, int, hipStream_t);
 void seq_launch_sandwich_residual(float*, const void*, const void*, const float*, const float*, const float*,
                                   const float*, void*, int, int, float, int, hipStream_t);
@@ -181,11 +188,11 @@ void latent_kv_store(torch::Tensor q, torch::Tensor dkv, torch::Tensor w, double
 // out [T, H, C] contiguous; q_abs [T, H, C] with free row and head strides;
 // q [T, H, D + R] row view; gate [T, H] row view or empty; tile_rows: rows per
 // workgroup of the matrix-unit kernel (0 = as many as fit), use_mfma false =
-// the plain kernel
+// the plain kernel; sink [H] fp32 or empty
 void attn_latent_paged(torch::Tensor out, torch::Tensor q_abs, torch::Tensor q, torch::Tensor cache,
                        torch::Tensor block_tables, torch::Tensor token_seg, torch::Tensor positions,
                        torch::Tensor gate, double scale, int64_t mask_size, int64_t nope_dim, int64_t tile_rows,
-                       bool use_mfma, torch::Tensor part_o, torch::Tensor part_ml) {
+                       bool use_mfma, torch::Tensor part_o, torch::Tensor part_ml, torch::Tensor sink) {
   CHECK_ACT(out); CHECK_ACT(q_abs); CHECK_SAME(q_abs, out); CHECK_ACT(q); CHECK_SAME(q, out); CHECK_ROWS3(q);
   CHECK_ACT(cache); CHECK_SAME(cache, out); CHECK_I32C(token_seg); CHECK_I64C(positions);
   TORCH_CHECK(block_tables.is_cuda() && block_tables.scalar_type() == at::kInt && block_tables.dim() == 2 &&
@@ -208,6 +215,8 @@ void attn_latent_paged(torch::Tensor out, torch::Tensor q_abs, torch::Tensor q, 
     nsplit = (int)part_o.size(2);
     TORCH_CHECK(nsplit >= 1 && nsplit <= 64 && part_ml.numel() == (int64_t)T * H * nsplit * 2);
   }
+  const bool has_sink = sink.numel() > 0;
+  if (has_sink) { CHECK_F32C(sink); TORCH_CHECK(sink.numel() == H); }
   if (T == 0) return;
   seq_launch_attn_latent_paged(out.data_ptr(), q_abs.data_ptr(), q.data_ptr(), cache.data_ptr(),
                                block_tables.data_ptr<int>(), token_seg.data_ptr<int>(),
@@ -215,8 +224,8 @@ void attn_latent_paged(torch::Tensor out, torch::Tensor q_abs, torch::Tensor q, 
                                (int)mask_size, T, H, D, R, C, (int)cache.size(2), (int)block_tables.stride(0),
                                q_abs.stride(0), q_abs.stride(1), (int)q.stride(0), g ? (int)gate.stride(0) : 0,
                                (int)tile_rows, use_mfma ? 1 : 0, nsplit > 1 ? part_o.data_ptr<float>() : nullptr,
-                               nsplit > 1 ? part_ml.data_ptr<float>() : nullptr, nsplit, f32flag(out),
-                               cur_stream());
+                               nsplit > 1 ? part_ml.data_ptr<float>() : nullptr, nsplit,
+                               has_sink ? sink.data_ptr<float>() : nullptr, f32flag(out), cur_stream());
 }
 
 void rmsnorm_cast(torch::Tensor out, torch::Tensor x, torch::Tensor w, double eps) {
@@ -257,17 +266,73 @@ void sandwich_residual(torch::Tensor x, torch::Tensor a, torch::Tensor b, torch:
                                want ? out.data_ptr() : nullptr, T, W, (float)eps, f32flag(a), cur_stream());
 }
 
-// gate_first: out = rms(o * silu(gate)) * w with w [G * S]; else out = rms(o) * w * sigmoid(gate) with w [S]
+// mode 0: out = rms(o) * w * sigmoid(gate), w [S]; 1: out = rms(o * silu(gate)) * w, w [G * S];
+// 2: out = rms(o) * w * silu(gate), w [S]; w empty = no weight
 void gated_rmsnorm(torch::Tensor out, torch::Tensor o, torch::Tensor w, torch::Tensor gate, double eps,
-                   bool gate_first) {
-  CHECK_ACT(out); CHECK_F32C(o); CHECK_F32C(w); CHECK_ACT(gate); CHECK_SAME(gate, out); CHECK_ROWS2(gate);
+                   int64_t mode) {
+  CHECK_ACT(out); CHECK_F32C(o); CHECK_ACT(gate); CHECK_SAME(gate, out); CHECK_ROWS2(gate);
+  TORCH_CHECK(mode >= 0 && mode <= 2, "gate mode");
   TORCH_CHECK(o.dim() == 3 && out.is_contiguous() && out.numel() == o.numel());
   const int T = o.size(0), G = o.size(1), S = o.size(2);
-  TORCH_CHECK(w.numel() == (gate_first ? (int64_t)G * S : S) && gate.size(0) == T &&
-              gate.size(1) == (int64_t)G * S);
+  const bool has_w = w.numel() > 0;
+  if (has_w) { CHECK_F32C(w); TORCH_CHECK(w.numel() == (mode == 1 ? (int64_t)G * S : S)); }
+  TORCH_CHECK(gate.size(0) == T && gate.size(1) == (int64_t)G * S);
   if (T == 0) return;
-  seq_launch_gated_rmsnorm(out.data_ptr(), o.data_ptr<float>(), w.data_ptr<float>(), gate.data_ptr(), T, G, S,
-                           (int)gate.stride(0), (float)eps, gate_first ? 1 : 0, f32flag(out), cur_stream());
+  seq_launch_gated_rmsnorm(out.data_ptr(), o.data_ptr<float>(), has_w ? w.data_ptr<float>() : nullptr,
+                           gate.data_ptr(), T, G, S, (int)gate.stride(0), (float)eps, (int)mode, f32flag(out),
+                           cur_stream());
+}
+
+// out = gelu(gate) * up
+void gelu_glu(torch::Tensor out, torch::Tensor gate, torch::Tensor up) {
+  CHECK_ACT(out); CHECK_ACT(gate); CHECK_SAME(up, gate); CHECK_SAME(out, gate); CHECK_ROWS2(gate); CHECK_ROWS2(up);
+  TORCH_CHECK(up.is_cuda() && up.sizes() == gate.sizes() && out.is_contiguous() && out.numel() == gate.numel());
+  if (gate.numel() == 0) return;
+  seq_launch_act_pair(out.data_ptr(), gate.data_ptr(), up.data_ptr(), nullptr, gate.size(0), (int)gate.size(1),
+                      (int)gate.size(1), (int)gate.stride(0), up.stride(0), 0, f32flag(gate), cur_stream());
+}
+
+// out = max(x, 0)^2
+void relu2(torch::Tensor out, torch::Tensor x) {
+  CHECK_ACT(out); CHECK_ACT(x); CHECK_SAME(out, x); CHECK_ROWS2(x);
+  TORCH_CHECK(out.is_contiguous() && out.numel() == x.numel());
+  if (x.numel() == 0) return;
+  seq_launch_act_pair(out.data_ptr(), x.data_ptr(), nullptr, nullptr, x.size(0), (int)x.size(1), (int)x.size(1),
+                      (int)x.stride(0), 0, 1, f32flag(x), cur_stream());
+}
+
+// x *= sigmoid(gate), element by element
+void sigmoid_gate(torch::Tensor x, torch::Tensor gate) {
+  CHECK_ACT(x); CHECK_ACT(gate); CHECK_SAME(gate, x); CHECK_ROWS2(x); CHECK_ROWS2(gate);
+  TORCH_CHECK(gate.sizes() == x.sizes());
+  if (x.numel() == 0) return;
+  seq_launch_act_pair(x.data_ptr(), x.data_ptr(), gate.data_ptr(), nullptr, x.size(0), (int)x.size(1),
+                      (int)x.stride(0), (int)x.stride(0), gate.stride(0), 2, f32flag(x), cur_stream());
+}
+
+// out = gelu(z) * table[ids, col0 : col0 + C]
+void gelu_mul_rows(torch::Tensor out, torch::Tensor z, torch::Tensor table, torch::Tensor ids, int64_t col0) {
+  CHECK_ACT(out); CHECK_ACT(z); CHECK_SAME(out, z); CHECK_ROWS2(z); CHECK_ACT(table); CHECK_SAME(table, z);
+  CHECK_I64C(ids);
+  const int T = z.size(0), C = z.size(1);
+  TORCH_CHECK(out.is_contiguous() && out.numel() == z.numel() && ids.numel() == T);
+  TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && col0 >= 0 && col0 + C <= table.size(1));
+  if (T == 0) return;
+  const char* base = (const char*)table.data_ptr() + col0 * table.element_size();
+  seq_launch_act_pair(out.data_ptr(), z.data_ptr(), base, ids.data_ptr<int64_t>(), T, C, C, (int)z.stride(0),
+                      table.size(1), 0, f32flag(z), cur_stream());
+}
+
+// x += a (+ b); out (may be empty) = x in the activation type
+void add_cast(torch::Tensor out, torch::Tensor x, torch::Tensor a, torch::Tensor b) {
+  CHECK_F32C(x); CHECK_ACT(a);
+  TORCH_CHECK(a.is_contiguous() && a.numel() == x.numel());
+  const bool has_b = b.numel() > 0, want = out.numel() > 0;
+  if (has_b) { CHECK_SAME(b, a); TORCH_CHECK(b.is_cuda() && b.is_contiguous() && b.numel() == x.numel()); }
+  if (want) { CHECK_SAME(out, a); TORCH_CHECK(out.is_cuda() && out.is_contiguous() && out.numel() == x.numel()); }
+  if (x.numel() == 0) return;
+  seq_launch_add_cast(want ? out.data_ptr() : nullptr, x.data_ptr<float>(), a.data_ptr(),
+                      has_b ? b.data_ptr() : nullptr, x.numel(), f32flag(a), cur_stream());
 }
 
 void gated_act(torch::Tensor out, torch::Tensor gate, torch::Tensor up, double limit, double alpha,
@@ -454,6 +519,28 @@ void linear_attn_decay(torch::Tensor o, torch::Tensor q, torch::Tensor k, torch:
                                cur_stream());
 }
 
+// q, k [T, H, D] and v [T, H, V] raw projections; rotation of the first 2 * inv_freq.numel() entries
+void retention(torch::Tensor o, torch::Tensor q, torch::Tensor k, torch::Tensor v, torch::Tensor decay,
+               torch::Tensor positions, torch::Tensor inv_freq, torch::Tensor state, torch::Tensor slots,
+               torch::Tensor cu, torch::Tensor seg_start) {
+  CHECK_F32C(o); CHECK_ACT(q); CHECK_ROWS3(q); CHECK_ROWS3(k); CHECK_ROWS3(v); CHECK_SAME(k, q); CHECK_SAME(v, q);
+  CHECK_F32C(decay); CHECK_F32C(state); CHECK_I64C(positions); CHECK_F32C(inv_freq);
+  check_segments(slots, cu, seg_start, state);
+  const int T = q.size(0), H = q.size(1), D = q.size(2), V = v.size(2), B = slots.numel(), R2 = inv_freq.numel();
+  TORCH_CHECK(k.is_cuda() && v.is_cuda() && k.size(0) == T && v.size(0) == T && k.size(1) == H &&
+              v.size(1) == H && k.size(2) == D && positions.numel() == T && 2 * R2 <= D);
+  TORCH_CHECK(D <= 256, "key size above 256 is not supported by the recurrence kernel");
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == D && state.size(3) == V);
+  TORCH_CHECK(decay.numel() == H && o.numel() == (int64_t)T * H * V);
+  if (T == 0 || B == 0) return;
+  auto packed = torch::empty({(int64_t)T, (int64_t)H * (2 * D + V)}, torch::dtype(torch::kFloat).device(q.device()));
+  seq_launch_retention(o.data_ptr<float>(), q.data_ptr(), k.data_ptr(), v.data_ptr(), decay.data_ptr<float>(),
+                       positions.data_ptr<int64_t>(), inv_freq.data_ptr<float>(), packed.data_ptr<float>(),
+                       state.data_ptr<float>(), slots.data_ptr<int>(), cu.data_ptr<int>(),
+                       seg_start.data_ptr<int>(), T, B, H, D, V, R2, (int)q.stride(0), (int)k.stride(0),
+                       (int)v.stride(0), f32flag(q), cur_stream());
+}
+
 void causal_conv_silu(torch::Tensor y, torch::Tensor x, torch::Tensor w, torch::Tensor conv_state,
                       torch::Tensor slots, torch::Tensor cu, torch::Tensor seg_start, torch::Tensor token_seg,
                       torch::Tensor bias) {
@@ -622,7 +709,7 @@ void moe_route(torch::Tensor idx, torch::Tensor w, torch::Tensor rowidx, torch::
   if (has_corr) CHECK_F32C(corr);
   const int T = x.size(0), N = fused ? router.size(0) : x.size(1);
   TORCH_CHECK(!has_corr || corr.numel() == N);
-  TORCH_CHECK(score_kind == 0 || score_kind == 1);
+  TORCH_CHECK(score_kind >= 0 && score_kind <= 2);
   int W = 0;
   if (fused) {
     CHECK_ACT(x); CHECK_F32C(router);
@@ -889,6 +976,12 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("moe_route", &moe_route);
   m.def("moe_combine", &moe_combine);
   m.def("gelu_tanh", &gelu_tanh);
+  m.def("gelu_glu", &gelu_glu);
+  m.def("relu2", &relu2);
+  m.def("sigmoid_gate", &sigmoid_gate);
+  m.def("gelu_mul_rows", &gelu_mul_rows);
+  m.def("add_cast", &add_cast);
+  m.def("retention", &retention);
   m.def("scale_softcap", &scale_softcap);
   m.def("scale_rows", &scale_rows);
   m.def("moe_spread_rows", &moe_spread_rows);

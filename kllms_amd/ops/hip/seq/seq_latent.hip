@@ -10,6 +10,8 @@
 //     - an MFMA kernel (bf16): 32 (row, head) query columns of one workgroup
 //       share each staged tile of 32 cached rows, for prompt portions,
 //       decoded tokens and mixes alike.
+// A sink (optional, one fp32 number per head) joins the softmax denominator as
+// exp(sink_h): the running maximum starts at it and the running sum at one.
 // Scores, softmax weights and the running sums are fp32 everywhere.
 
 #include "seq_common.h"
@@ -68,7 +70,7 @@ __global__ void attn_latent_paged_kernel(T* __restrict__ out, const T* __restric
                                          const int64_t* __restrict__ positions, const T* __restrict__ gate,
                                          float scale, int mask_size, int H, int D, int R, int C, int BS,
                                          int bt_stride, int64_t qa_stride_t, int64_t qa_stride_h, int q_stride,
-                                         int gate_stride) {
+                                         int gate_stride, const float* __restrict__ sink) {
   extern __shared__ float lds[];       // query [C + R] | weights [64] | cache row index [64] (as int)
   const int L = C + R;
   float* qs = lds;
@@ -88,7 +90,7 @@ __global__ void attn_latent_paged_kernel(T* __restrict__ out, const T* __restric
   float acc[LAT_MAX_ACC];
 #pragma unroll
   for (int i = 0; i < LAT_MAX_ACC; ++i) acc[i] = 0.f;
-  float m = -INFINITY, l = 0.f;
+  float m = sink != nullptr ? sink[h] : -INFINITY, l = sink != nullptr ? 1.f : 0.f;
   for (int base = 0; base < total; base += WAVE) {
     const int u = base + lane;
     float s = -INFINITY;
@@ -103,7 +105,7 @@ __global__ void attn_latent_paged_kernel(T* __restrict__ out, const T* __restric
     }
     const float m_new = fmaxf(m, wave_max(s));
     const float w = u < total ? expf(s - m_new) : 0.f;
-    const float corr = expf(m - m_new);        // m = -inf on the first tile -> 0
+    const float corr = expf(m - m_new);        // without a sink m = -inf on the first tile -> 0
     l = l * corr + wave_sum(w);
     m = m_new;
     ps[lane] = w;
@@ -202,7 +204,7 @@ __global__ void __launch_bounds__(WAVE * LAT_WAVES, 2) attn_latent_mfma_kernel(
     const int64_t* __restrict__ positions, const bfraw* __restrict__ gate, float scale, int mask_size, int T_,
     int H, int D, int R, int C, int BS, int bt_stride, int64_t qa_stride_t, int64_t qa_stride_h, int q_stride,
     int gate_stride, int tile_rows, int hb, int vec, int qvec, float* __restrict__ part_o,
-    float* __restrict__ part_ml) {
+    float* __restrict__ part_ml, const float* __restrict__ sink) {
   extern __shared__ __align__(16) unsigned char lat_smem[];
   const int L = C + R;
   const int Lp = (L + 15) / 16 * 16;
@@ -278,6 +280,11 @@ __global__ void __launch_bounds__(WAVE * LAT_WAVES, 2) attn_latent_mfma_kernel(
     for (int r = 0; r < 16; ++r) o_acc[i][r] = 0.f;
   float m_run = -INFINITY, l_run = 0.f;
   const float scale2 = scale * 1.4426950408889634f;
+  // the sink counts once per column: in the first key share, in one lane of the column's pair
+  if (sink != nullptr && cvalid && blockIdx.z == 0) {
+    m_run = sink[chead] * 1.4426950408889634f;
+    l_run = half == 0 ? 1.f : 0.f;
+  }
 
   // one pass per sequence present in the tile (rows are packed by sequence)
   int ra = 0;
@@ -555,8 +562,8 @@ extern "C" void seq_launch_attn_latent_paged(void* out, const void* q_abs, const
                                              int mask_size, int T_, int H, int D, int R, int C, int BS,
                                              int bt_stride, int64_t qa_stride_t, int64_t qa_stride_h,
                                              int q_stride, int gate_stride, int tile_rows, int use_mfma,
-                                             float* part_o, float* part_ml, int nsplit, int is_f32,
-                                             hipStream_t st) {
+                                             float* part_o, float* part_ml, int nsplit, const float* sink,
+                                             int is_f32, hipStream_t st) {
   const int L = C + R;
   if (use_mfma && !is_f32 && L <= 16 * LAT_WAVES * LAT_MAX_SL && C <= 32 * LAT_WAVES * LAT_MAX_DT) {
     int hb = 1;
@@ -573,7 +580,7 @@ extern "C" void seq_launch_attn_latent_paged(void* out, const void* q_abs, const
                        dim3(WAVE * LAT_WAVES), lds, st, (bfraw*)out, (const bfraw*)q_abs, (const bfraw*)q,
                        (const bfraw*)cache, block_tables, token_seg, positions, (const bfraw*)gate, scale,
                        mask_size, T_, H, D, R, C, BS, bt_stride, qa_stride_t, qa_stride_h, q_stride, gate_stride,
-                       tr, hb, vec, qvec, part_o, part_ml);
+                       tr, hb, vec, qvec, part_o, part_ml, sink);
     if (ns > 1)
       hipLaunchKernelGGL(attn_latent_merge_kernel, dim3(T_, H), dim3(256), 0, st, (bfraw*)out, part_o, part_ml,
                          (const bfraw*)gate, H, C, ns, gate_stride);
@@ -583,5 +590,5 @@ extern "C" void seq_launch_attn_latent_paged(void* out, const void* q_abs, const
   DISPATCH_T(is_f32, hipLaunchKernelGGL(attn_latent_paged_kernel<T>, dim3(T_, H), dim3(WAVE), lds, st, (T*)out,
                                         (const T*)q_abs, (const T*)q, (const T*)cache, block_tables, token_seg,
                                         positions, (const T*)gate, scale, mask_size, H, D, R, C, BS, bt_stride,
-                                        qa_stride_t, qa_stride_h, q_stride, gate_stride);)
+                                        qa_stride_t, qa_stride_h, q_stride, gate_stride, sink);)
 }

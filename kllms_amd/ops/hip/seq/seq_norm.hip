@@ -158,13 +158,27 @@ __global__ void sandwich_residual_v8_kernel(float* __restrict__ x, const T* __re
   }
 }
 
-// out[t, g*S + i] = o[t,g,i] / rms(o[t,g,:]) * w[i] * sigmoid(gate[t, g*S + i])
-// gate_first: the gate is silu and comes before the norm, the weight spans the
-// whole row: y = o * silu(gate); out = y / rms(y[t,g,:]) * w[g*S + i]
+// Gate modes of the grouped norms:
+//   GATE_SIGMOID     out[t, g*S + i] = o[t,g,i] / rms(o[t,g,:]) * w[i] * sigmoid(gate[t, g*S + i])
+//   GATE_SILU_FIRST  the gate comes before the norm, the weight spans the whole
+//                    row: y = o * silu(gate); out = y / rms(y[t,g,:]) * w[g*S + i]
+//   GATE_SILU        as GATE_SIGMOID with silu
+// w == nullptr: no weight.
+#define GATE_SIGMOID 0
+#define GATE_SILU_FIRST 1
+#define GATE_SILU 2
+__device__ __forceinline__ float gate_after(float g, int mode) {
+  return mode == GATE_SIGMOID ? sigmoid_exact(g) : silu_exact(g);
+}
+__device__ __forceinline__ void ld_weight8(const float* w, int64_t i, float v[8]) {
+  if (w != nullptr) { ld8(w + i, v); return; }
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v[e] = 1.0f;
+}
 template <typename T>
 __global__ void gated_rmsnorm_kernel(T* __restrict__ out, const float* __restrict__ o,
                                      const float* __restrict__ w, const T* __restrict__ gate,
-                                     int S, int gate_stride, float eps, int gate_first) {
+                                     int S, int gate_stride, float eps, int mode) {
   __shared__ float scratch[16];
   const int t = blockIdx.x, g = blockIdx.y, G = gridDim.y;
   const float* row = o + ((int64_t)t * G + g) * S;
@@ -172,7 +186,7 @@ __global__ void gated_rmsnorm_kernel(T* __restrict__ out, const float* __restric
   float ss = 0.f;
   for (int i = threadIdx.x; i < S; i += blockDim.x) {
     float v = row[i];
-    if (gate_first) v *= silu_exact(ldf(grow + i));
+    if (mode == GATE_SILU_FIRST) v *= silu_exact(ldf(grow + i));
     ss += v * v;
   }
   ss = block_sum(ss, scratch);
@@ -180,8 +194,8 @@ __global__ void gated_rmsnorm_kernel(T* __restrict__ out, const float* __restric
   T* orow = out + ((int64_t)t * G + g) * S;
   for (int i = threadIdx.x; i < S; i += blockDim.x) {
     const float gv = ldf(grow + i);
-    stf(orow + i, gate_first ? row[i] * silu_exact(gv) * r * w[(int64_t)g * S + i]
-                             : row[i] * r * w[i] * sigmoid_exact(gv));
+    const float wv = w == nullptr ? 1.0f : w[(mode == GATE_SILU_FIRST ? (int64_t)g * S : 0) + i];
+    stf(orow + i, mode == GATE_SILU_FIRST ? row[i] * silu_exact(gv) * r * wv : row[i] * r * wv * gate_after(gv, mode));
   }
 }
 
@@ -190,7 +204,7 @@ __global__ void gated_rmsnorm_kernel(T* __restrict__ out, const float* __restric
 template <typename T>
 __global__ void gated_rmsnorm_v8_kernel(T* __restrict__ out, const float* __restrict__ o,
                                         const float* __restrict__ w, const T* __restrict__ gate,
-                                        int S, int gate_stride, float eps, int gate_first) {
+                                        int S, int gate_stride, float eps, int mode) {
   __shared__ float scratch[16];
   const int t = blockIdx.x, g = blockIdx.y, G = gridDim.y;
   const float* row = o + ((int64_t)t * G + g) * S;
@@ -202,7 +216,7 @@ __global__ void gated_rmsnorm_v8_kernel(T* __restrict__ out, const float* __rest
     const int i = (threadIdx.x + c * blockDim.x) * 8;
     if (i < S) {
       ld8(row + i, v[c]);
-      if (gate_first) {
+      if (mode == GATE_SILU_FIRST) {
         ld8(grow + i, gg);
 #pragma unroll
         for (int e = 0; e < 8; ++e) v[c][e] *= silu_exact(gg[e]);
@@ -218,14 +232,13 @@ __global__ void gated_rmsnorm_v8_kernel(T* __restrict__ out, const float* __rest
   for (int c = 0; c < 2; ++c) {
     const int i = (threadIdx.x + c * blockDim.x) * 8;
     if (i < S) {
-      if (gate_first) {
-        ld8(w + (int64_t)g * S + i, ww);
+      ld_weight8(w, (mode == GATE_SILU_FIRST ? (int64_t)g * S : 0) + i, ww);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) v[c][e] = v[c][e] * r * ww[e];
-      } else {
-        ld8(w + i, ww); ld8(grow + i, gg);
+      for (int e = 0; e < 8; ++e) v[c][e] = v[c][e] * r * ww[e];
+      if (mode != GATE_SILU_FIRST) {
+        ld8(grow + i, gg);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) v[c][e] = v[c][e] * r * ww[e] * sigmoid_exact(gg[e]);
+        for (int e = 0; e < 8; ++e) v[c][e] *= gate_after(gg[e], mode);
       }
       st8(orow + i, v[c]);
     }
@@ -238,7 +251,7 @@ template <typename T>
 __global__ void gated_rmsnorm_rows_kernel(T* __restrict__ out, const float* __restrict__ o,
                                           const float* __restrict__ w, const T* __restrict__ gate,
                                           int64_t rows, int G, int S, int LPG, int gate_stride, float eps,
-                                          int gate_first) {
+                                          int mode) {
   const int64_t tid = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
   const int64_t row = tid / LPG;
   const int i = (int)(tid - row * LPG) * 8;
@@ -250,7 +263,7 @@ __global__ void gated_rmsnorm_rows_kernel(T* __restrict__ out, const float* __re
   if (on) {
     ld8(o + row * S + i, v);
     ld8(gate + t * gate_stride + (int64_t)g * S + i, gg);
-    if (gate_first) {
+    if (mode == GATE_SILU_FIRST) {
 #pragma unroll
       for (int e = 0; e < 8; ++e) v[e] *= silu_exact(gg[e]);
     }
@@ -260,9 +273,9 @@ __global__ void gated_rmsnorm_rows_kernel(T* __restrict__ out, const float* __re
   for (int off = 1; off < LPG; off <<= 1) ss += __shfl_xor(ss, off);
   if (!on) return;
   const float r = 1.0f / sqrtf(ss / (float)S + eps);
-  ld8(w + (gate_first ? (int64_t)g * S : 0) + i, ww);
+  ld_weight8(w, (mode == GATE_SILU_FIRST ? (int64_t)g * S : 0) + i, ww);
 #pragma unroll
-  for (int e = 0; e < 8; ++e) v[e] = v[e] * r * ww[e] * (gate_first ? 1.0f : sigmoid_exact(gg[e]));
+  for (int e = 0; e < 8; ++e) v[e] = v[e] * r * ww[e] * (mode == GATE_SILU_FIRST ? 1.0f : gate_after(gg[e], mode));
   st8(out + row * S + i, v);
 }
 
@@ -328,6 +341,44 @@ __global__ void gelu_tanh_v8_kernel(T* __restrict__ out, const T* __restrict__ x
   }
 }
 
+// Elementwise activations of row views, in fp32 between load and store:
+//   ACT_GELU_MUL    out = gelu(a) * b                (gated gelu feed-forward; a token's side row)
+//   ACT_RELU2       out = max(a, 0)^2
+//   ACT_SIGMOID_MUL out = a * sigmoid(b)
+// Row r of b is b + r * b_stride, or with ids b + ids[r] * b_stride (b then
+// already points at its first column). gelu in the form z * sigmoid(2 u), equal
+// to z (1 + tanh(u)) / 2.
+#define ACT_GELU_MUL 0
+#define ACT_RELU2 1
+#define ACT_SIGMOID_MUL 2
+template <int OP>
+__device__ __forceinline__ float act_pair(float a, float b) {
+  if (OP == ACT_GELU_MUL) return a * sigmoid_exact(1.5957691216057308f * (a + 0.044715f * a * a * a)) * b;
+  if (OP == ACT_RELU2) { const float p = fmaxf(a, 0.f); return p * p; }
+  return a * sigmoid_exact(b);
+}
+
+template <typename T, int OP, int VEC>
+__global__ void act_pair_kernel(T* __restrict__ out, const T* a, const T* __restrict__ b,
+                                const int64_t* __restrict__ ids, int64_t n, int cols, int out_stride, int a_stride,
+                                int64_t b_stride) {
+  const int cv = cols / VEC;
+  for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (int64_t)gridDim.x * blockDim.x) {
+    const int64_t r = i / cv, c = (i - r * cv) * VEC;
+    const T* br = OP == ACT_RELU2 ? nullptr : b + (ids != nullptr ? ids[r] : r) * b_stride + c;
+    if (VEC == 8) {
+      float av[8], bv[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      ld8(a + r * a_stride + c, av);
+      if (OP != ACT_RELU2) ld8(br, bv);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) av[e] = act_pair<OP>(av[e], bv[e]);
+      st8(out + r * out_stride + c, av);
+    } else {
+      stf(out + r * out_stride + c, act_pair<OP>(ldf(a + r * a_stride + c), OP == ACT_RELU2 ? 0.f : ldf(br)));
+    }
+  }
+}
+
 // z <- z * scale, then cap * tanh(z / cap) when cap > 0 (fp32 logits, in place)
 __global__ void scale_softcap_kernel(float* __restrict__ z, int64_t n, float scale, float cap) {
   for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n;
@@ -360,6 +411,32 @@ extern "C" void seq_launch_gelu_tanh(void* out, const void* x, int64_t rows, int
   const int grid = (int)((n + 255) / 256 < 4096 ? (n + 255) / 256 : 4096);
   DISPATCH_T(is_f32, hipLaunchKernelGGL(gelu_tanh_kernel<T>, dim3(grid), dim3(256), 0, st, (T*)out, (const T*)x,
                                         n, cols, stride);)
+}
+
+template <typename T, int OP>
+static void launch_act_pair(void* out, const void* a, const void* b, const int64_t* ids, int64_t rows, int cols,
+                            int out_stride, int a_stride, int64_t b_stride, hipStream_t st) {
+  const bool v8 = cols % 8 == 0 && out_stride % 8 == 0 && a_stride % 8 == 0 && b_stride % 8 == 0 && aligned16(out) &&
+                  aligned16(a) && (b == nullptr || aligned16(b));
+  const int64_t n = rows * cols / (v8 ? 8 : 1);
+  const int grid = (int)((n + 255) / 256 < 16384 ? (n + 255) / 256 : 16384);
+  if (v8) hipLaunchKernelGGL((act_pair_kernel<T, OP, 8>), dim3(grid), dim3(256), 0, st, (T*)out, (const T*)a,
+                             (const T*)b, ids, n, cols, out_stride, a_stride, b_stride);
+  else hipLaunchKernelGGL((act_pair_kernel<T, OP, 1>), dim3(grid), dim3(256), 0, st, (T*)out, (const T*)a,
+                          (const T*)b, ids, n, cols, out_stride, a_stride, b_stride);
+}
+
+// op: ACT_*; ids: row indices into b, or nullptr
+extern "C" void seq_launch_act_pair(void* out, const void* a, const void* b, const int64_t* ids, int64_t rows,
+                                    int cols, int out_stride, int a_stride, int64_t b_stride, int op, int is_f32,
+                                    hipStream_t st) {
+  DISPATCH_T(is_f32,
+             if (op == ACT_GELU_MUL)
+               launch_act_pair<T, ACT_GELU_MUL>(out, a, b, ids, rows, cols, out_stride, a_stride, b_stride, st);
+             else if (op == ACT_RELU2)
+               launch_act_pair<T, ACT_RELU2>(out, a, b, ids, rows, cols, out_stride, a_stride, b_stride, st);
+             else
+               launch_act_pair<T, ACT_SIGMOID_MUL>(out, a, b, ids, rows, cols, out_stride, a_stride, b_stride, st);)
 }
 
 extern "C" void seq_launch_scale_softcap(float* z, int64_t n, float scale, float cap, hipStream_t st) {
@@ -396,28 +473,28 @@ extern "C" void seq_launch_sandwich_residual(float* x, const void* a, const void
 }
 
 extern "C" void seq_launch_gated_rmsnorm(void* out, const float* o, const float* w, const void* gate,
-                                         int T_, int G, int S, int gate_stride, float eps, int gate_first,
+                                         int T_, int G, int S, int gate_stride, float eps, int mode,
                                          int is_f32, hipStream_t st) {
-  if (S % 8 == 0 && gate_stride % 8 == 0 && aligned16(out) && aligned16(o) && aligned16(w) && aligned16(gate)) {
+  if (S % 8 == 0 && gate_stride % 8 == 0 && aligned16(out) && aligned16(o) && (w == nullptr || aligned16(w)) && aligned16(gate)) {
     const int lpg = S / 8;
     if (lpg <= 64 && (lpg & (lpg - 1)) == 0) {
       const int64_t rows = (int64_t)T_ * G;
       const int grid = (int)((rows * lpg + 255) / 256);
       DISPATCH_T(is_f32, hipLaunchKernelGGL(gated_rmsnorm_rows_kernel<T>, dim3(grid), dim3(256), 0, st, (T*)out,
-                                            o, w, (const T*)gate, rows, G, S, lpg, gate_stride, eps, gate_first);)
+                                            o, w, (const T*)gate, rows, G, S, lpg, gate_stride, eps, mode);)
       return;
     }
     int threads = ((lpg + 1) / 2 + WAVE - 1) / WAVE * WAVE;       // two chunks of 8 per thread
     if (threads <= 1024) {
       if (threads < WAVE) threads = WAVE;
       DISPATCH_T(is_f32, hipLaunchKernelGGL(gated_rmsnorm_v8_kernel<T>, dim3(T_, G), dim3(threads), 0, st,
-                                            (T*)out, o, w, (const T*)gate, S, gate_stride, eps, gate_first);)
+                                            (T*)out, o, w, (const T*)gate, S, gate_stride, eps, mode);)
       return;
     }
   }
   const int threads = S >= 256 ? 256 : (S > 64 ? 128 : 64);
   DISPATCH_T(is_f32, hipLaunchKernelGGL(gated_rmsnorm_kernel<T>, dim3(T_, G), dim3(threads), 0, st, (T*)out,
-                                        o, w, (const T*)gate, S, gate_stride, eps, gate_first);)
+                                        o, w, (const T*)gate, S, gate_stride, eps, mode);)
 }
 
 extern "C" void seq_launch_gated_act(void* out, const void* gate, const void* up, int64_t rows, int cols,

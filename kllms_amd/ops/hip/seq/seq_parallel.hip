@@ -163,6 +163,28 @@ __global__ void cast_concat_kernel(T* __restrict__ out, float* __restrict__ x, c
   }
 }
 
+// ---- x += a (+ b), out = x in the activation type (out == nullptr: none) ----------
+template <typename T, int VEC>
+__global__ void add_cast_kernel(T* __restrict__ out, float* __restrict__ x, const T* __restrict__ a,
+                                const T* __restrict__ b, int64_t n) {
+  for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < n; i += (int64_t)gridDim.x * blockDim.x) {
+    if (VEC == 8) {
+      float v[8], u[8], w[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      ld8(x + i * 8, v);
+      ld8(a + i * 8, u);
+      if (b != nullptr) ld8(b + i * 8, w);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] += u[e] + w[e];
+      st8(x + i * 8, v);
+      if (out != nullptr) st8(out + i * 8, v);
+    } else {
+      const float v = x[i] + (ldf(a + i) + (b != nullptr ? ldf(b + i) : 0.f));
+      x[i] = v;
+      if (out != nullptr) stf(out + i, v);
+    }
+  }
+}
+
 // ---- per-head RMS norm, full-width weight, activated gate ------------------------
 // o [T, H, S] fp32; out[t, h*S + i] = o / rms(o[t,h,:]) * w[h*S + i] * act(gate[t, h*S + i]);
 // act = sigmoid (0) or silu (1). One wave per (row, head). With mt != nullptr the
@@ -260,7 +282,10 @@ __global__ void shift_state_update_kernel(const T* __restrict__ h, T* __restrict
 }
 
 // ---- router --------------------------------------------------------------------
-// One workgroup per row (the routing proper is its first wave's). s = softmax(z) over the N outputs; c = s + correction; the
+// One workgroup per row (the routing proper is its first wave's). Scores by
+// score_kind: 0 = softmax(z) over the N outputs, 1 = sigmoid(z), 2 = exp(z - max z);
+// c = s + correction (kind 2: z + correction, so the choice is made on the
+// logits and renormalised weights are the softmax over the chosen ones); the
 // outputs form `gc` equal groups of neighbours, a group's score is its largest
 // c, the best `gk` groups stay eligible; the `top` eligible outputs with the
 // largest c are chosen (ties: the lower index). w = chosen s / (sum + 1e-20).
@@ -314,6 +339,14 @@ __global__ void __launch_bounds__(256) moe_route_kernel(int* __restrict__ idx, f
     for (int e = lane; e < N; e += WAVE) { const float p = expf(zs[e] - mx); ss[e] = p; sum += p; }
     sum = wave_sum(sum);
     for (int e = lane; e < N; e += WAVE) { ss[e] /= sum; cs[e] = ss[e] + (corr != nullptr ? corr[e] : 0.f); }
+  } else if (wave == 0 && score_kind == 2) {   // choice by the logits, weights relative to the largest
+    float mx = -INFINITY;
+    for (int e = lane; e < N; e += WAVE) mx = fmaxf(mx, zs[e]);
+    mx = wave_max(mx);
+    for (int e = lane; e < N; e += WAVE) {
+      ss[e] = expf(zs[e] - mx);
+      cs[e] = zs[e] + (corr != nullptr ? corr[e] : 0.f);
+    }
   } else if (wave == 0) {                      // sigmoid of each output
     for (int e = lane; e < N; e += WAVE) {
       ss[e] = sigmoid_exact(zs[e]);
@@ -500,6 +533,19 @@ extern "C" void seq_launch_cast_concat(void* out, float* x, const float* x0, con
                                        int T_, int W, int is_f32, hipStream_t st) {
   DISPATCH_T(is_f32, hipLaunchKernelGGL(cast_concat_kernel<T>, dim3(T_), dim3(row_threads(W)), 0, st, (T*)out, x,
                                         x0, (const T*)a, (const T*)b, W);)
+}
+
+extern "C" void seq_launch_add_cast(void* out, float* x, const void* a, const void* b, int64_t n, int is_f32,
+                                    hipStream_t st) {
+  const bool v8 = n % 8 == 0 && aligned16(x) && aligned16(a) && (b == nullptr || aligned16(b)) &&
+                  (out == nullptr || aligned16(out));
+  const int64_t m = v8 ? n / 8 : n;
+  const int grid = (int)((m + 255) / 256 < 16384 ? (m + 255) / 256 : 16384);
+  DISPATCH_T(is_f32,
+             if (v8) hipLaunchKernelGGL((add_cast_kernel<T, 8>), dim3(grid), dim3(256), 0, st, (T*)out, x, (const T*)a,
+                                        (const T*)b, m);
+             else hipLaunchKernelGGL((add_cast_kernel<T, 1>), dim3(grid), dim3(256), 0, st, (T*)out, x, (const T*)a,
+                                     (const T*)b, m);)
 }
 
 extern "C" void seq_launch_head_rmsnorm_gate(void* out, const float* o, const float* w, const void* gate,

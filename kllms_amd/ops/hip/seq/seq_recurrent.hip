@@ -176,6 +176,53 @@ __global__ void __launch_bounds__(WAVE) linear_attn_decay_kernel(
   }
 }
 
+// ---- retention: the same recurrence on rotated q and k ----------------------------
+// Pre-pass, one workgroup per token: sin / cos of the token's angles
+// (float(pos) * inv_freq[i]) once in LDS, then per head in the packed layout
+// [rot(q) (D) | rot(k) * D^-1/2 (D) | v (V)], fp32. Entry i of the first 2 R2
+// rotates with entry i + R2. VEC = 8: D, V, R2 and the strides are multiples of 8.
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256) retention_prep_kernel(
+    float* __restrict__ pk, const T* __restrict__ q, const T* __restrict__ k, const T* __restrict__ v,
+    const int64_t* __restrict__ positions, const float* __restrict__ inv_freq, float kscale, int H, int D, int V,
+    int R2, int q_stride, int k_stride, int v_stride) {
+  extern __shared__ __align__(16) float cs[];          // cos [R2] | sin [R2]
+  const int64_t t = blockIdx.x;
+  const float pos = (float)positions[t];
+  for (int i = threadIdx.x; i < R2; i += blockDim.x) sincosf(pos * inv_freq[i], &cs[R2 + i], &cs[i]);
+  __syncthreads();
+  const int W = 2 * D + V, WV = W / VEC;
+  for (int u = threadIdx.x; u < H * WV; u += blockDim.x) {
+    const int h = u / WV, c = (u - h * WV) * VEC;
+    float x[VEC], y[VEC], cc[VEC], sn[VEC];
+    auto load = [&](const T* p, float* d) {
+      if constexpr (VEC == 8) ld8(p, d); else d[0] = ldf(p);
+    };
+    if (c >= 2 * D) {
+      load(v + t * v_stride + (int64_t)h * V + (c - 2 * D), x);
+    } else {
+      const bool isk = c >= D;
+      const int d = isk ? c - D : c;
+      const T* row = (isk ? k + t * k_stride : q + t * q_stride) + (int64_t)h * D;
+      load(row + d, x);
+      if (d < 2 * R2) {
+        const bool lo = d < R2;
+        const int i = lo ? d : d - R2;
+        load(row + (lo ? d + R2 : d - R2), y);
+        if constexpr (VEC == 8) { ld8(cs + i, cc); ld8(cs + R2 + i, sn); } else { cc[0] = cs[i]; sn[0] = cs[R2 + i]; }
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) x[e] = x[e] * cc[e] + (lo ? -y[e] : y[e]) * sn[e];
+      }
+      if (isk) {
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) x[e] *= kscale;
+      }
+    }
+    float* dst = pk + (t * H + h) * W + c;
+    if constexpr (VEC == 8) st8(dst, x); else dst[0] = x[0];
+  }
+}
+
 // ---- short causal convolution + silu ----------------------------------------
 // y[t,c] = silu(bias[c] + sum_j w[j,c] * x[t - (K-1-j), c]) (bias optional; weights taps-major [K, C],
 // last tap = current token); inputs before the segment
@@ -483,6 +530,29 @@ extern "C" void seq_launch_linear_attn_decay(float* o, const void* q, const void
                                           (const T*)q, (const T*)k, (const T*)v, n, H, D, V, q_stride, k_stride,
                                           v_stride);)
   }
+  const int ns = pick_split(B, H, V);
+  DISPATCH_NS(ns, DISPATCH_D(D, hipLaunchKernelGGL((linear_attn_decay_kernel<DMAX, NS>),
+                                                   dim3(B, H, (V + WAVE / NS - 1) / (WAVE / NS)), dim3(WAVE), 0,
+                                                   st, o, packed, decay, nullptr, nullptr, state, slots, cu,
+                                                   seg_start, H, D, V);))
+}
+
+extern "C" void seq_launch_retention(float* o, const void* q, const void* k, const void* v, const float* decay,
+                                     const int64_t* positions, const float* inv_freq, float* packed, float* state,
+                                     const int* slots, const int* cu, const int* seg_start, int T_, int B, int H,
+                                     int D, int V, int R2, int q_stride, int k_stride, int v_stride, int is_f32,
+                                     hipStream_t st) {
+  const float kscale = 1.0f / sqrtf((float)D);
+  const size_t lds = (size_t)2 * (R2 > 0 ? R2 : 1) * sizeof(float);
+  const bool v8 = D % 8 == 0 && V % 8 == 0 && R2 % 8 == 0 && q_stride % 8 == 0 && k_stride % 8 == 0 &&
+                  v_stride % 8 == 0 && aligned16(q) && aligned16(k) && aligned16(v) && aligned16(packed);
+  DISPATCH_T(is_f32,
+             if (v8) hipLaunchKernelGGL((retention_prep_kernel<T, 8>), dim3(T_), dim3(256), lds, st, packed,
+                                        (const T*)q, (const T*)k, (const T*)v, positions, inv_freq, kscale, H, D, V,
+                                        R2, q_stride, k_stride, v_stride);
+             else hipLaunchKernelGGL((retention_prep_kernel<T, 1>), dim3(T_), dim3(256), lds, st, packed,
+                                     (const T*)q, (const T*)k, (const T*)v, positions, inv_freq, kscale, H, D, V,
+                                     R2, q_stride, k_stride, v_stride);)
   const int ns = pick_split(B, H, V);
   DISPATCH_NS(ns, DISPATCH_D(D, hipLaunchKernelGGL((linear_attn_decay_kernel<DMAX, NS>),
                                                    dim3(B, H, (V + WAVE / NS - 1) / (WAVE / NS)), dim3(WAVE), 0,

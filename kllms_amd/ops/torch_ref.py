@@ -380,14 +380,18 @@ def linear_attn_decay(q, k, v, decay, state, state_slots, cu_seqlens, seg_start)
     return o
 
 
-def gated_rmsnorm(o, weight, gate, eps, out_dtype) -> torch.Tensor:
+def gated_rmsnorm(o, weight, gate, eps, out_dtype, gate_act="sigmoid") -> torch.Tensor:
     """o [T, n_groups, S] fp32: each group is divided by its root mean square,
-    times weight [S], times sigmoid(gate) ([T, n_groups*S] logits).
-    Returns [T, n_groups*S]."""
+    times weight [S] (None = ones), times sigmoid(gate) or silu(gate)
+    ([T, n_groups*S] logits). Returns [T, n_groups*S]."""
     T, Gn, S = o.shape
     of = o.float()
-    y = of * torch.rsqrt(of.pow(2).mean(-1, keepdim=True) + eps) * weight.float()
-    return (y.reshape(T, Gn * S) * torch.sigmoid(gate.float())).to(out_dtype)
+    y = of * torch.rsqrt(of.pow(2).mean(-1, keepdim=True) + eps)
+    if weight is not None:
+        y = y * weight.float()
+    gf = gate.float()
+    gf = torch.sigmoid(gf) if gate_act == "sigmoid" else torch.nn.functional.silu(gf)
+    return (y.reshape(T, Gn * S) * gf).to(out_dtype)
 
 
 def causal_conv_silu(x, w, conv_state, state_slots, cu_seqlens, seg_start, bias=None) -> torch.Tensor:
@@ -666,15 +670,20 @@ def gated_act(gate, up, limit: float, alpha: float, up_bias: float) -> torch.Ten
 
 
 def moe_route(z, correction, top, group_count, group_keep, score="softmax", renormalize=True):
-    """z [T, N] fp32 router logits. Scores s = softmax(z) over the outputs, or
-    sigmoid(z) of each; the choice is made on c = s + correction (None = no
-    correction) among the experts of the ``group_keep`` groups (of
+    """z [T, N] fp32 router logits. Scores s = softmax(z) over the outputs,
+    sigmoid(z) of each, or ("top_softmax") exp(z - max z); the choice is made
+    on c = s + correction (None = no correction; "top_softmax": on z + correction) among the experts of the ``group_keep`` groups (of
     ``group_count`` equal runs of neighbours) whose largest c is largest;
     ties go to the lower index. Returns (idx [T, top] int32, w [T, top] fp32
     = chosen s, divided by (their sum + 1e-20) if ``renormalize``)."""
     T, N = z.shape
-    s = torch.softmax(z.float(), -1) if score == "softmax" else torch.sigmoid(z.float())
-    c = s + correction.float() if correction is not None else s
+    zf = z.float()
+    if score == "top_softmax":
+        s, c = torch.exp(zf - zf.max(-1, keepdim=True).values), zf
+    else:
+        c = s = torch.softmax(zf, -1) if score == "softmax" else torch.sigmoid(zf)
+    if correction is not None:
+        c = c + correction.float()
     per = N // group_count
     gs = c.view(T, group_count, per).max(-1).values
     # stable descending order = ties to the lower index
@@ -766,14 +775,15 @@ def latent_kv_store(q, dkv, w_norm, eps, positions, inv_freq, cache, slot_mappin
 
 
 def attn_latent_paged(q_abs, q, cache, block_tables, token_seg, positions, scale, mask_size, gate,
-                      nope_dim, out_dtype=None) -> torch.Tensor:
+                      nope_dim, sink=None, out_dtype=None) -> torch.Tensor:
     """Latent attention in its absorbed form. q_abs [T, H, C]: the unrotated
     query parts already multiplied into the latent space; q [T, H, nope_dim +
     R]: its last R entries are the rotated query parts. cache [NB, 1, BS,
     C + R] rows [latent | rotated key part]. Row t at position p sees keys j
     of its own sequence with 0 <= p - j < mask_size (0 = all j <= p):
       score = (q_abs . latent_j + q_rot . krot_j) * scale,  softmax in fp32,
-      out[t, h] = sum_j weight_j latent_j   (times sigmoid(gate[t, h]))."""
+      out[t, h] = sum_j weight_j latent_j   (times sigmoid(gate[t, h])).
+    sink [H] fp32 (None = none): the softmax denominator also holds exp(sink_h)."""
     T, H, C = q_abs.shape
     BS = cache.shape[2]
     out = torch.empty(T, H, C, dtype=out_dtype or q.dtype, device=q.device)
@@ -784,11 +794,77 @@ def attn_latent_paged(q_abs, q, cache, block_tables, token_seg, positions, scale
         idx = torch.arange(lo, p + 1, device=q.device)
         rows = cache[block_tables[seg[t]].long()[idx // BS], 0, idx % BS].float()        # [n, C+R]
         s = (q_abs[t].float() @ rows[:, :C].T + q[t, :, nope_dim:].float() @ rows[:, C:].T) * scale
-        o = torch.softmax(s, -1) @ rows[:, :C]
+        if sink is None:
+            pr = torch.softmax(s, -1)
+        else:
+            pr = torch.softmax(torch.cat([s, sink.float()[:, None]], -1), -1)[:, :-1]
+        o = pr @ rows[:, :C]
         if gate is not None:
             o = o * torch.sigmoid(gate[t].float())[:, None]
         out[t] = o.to(out.dtype)
     return out
+
+
+def sigmoid_gate_(x, gate) -> None:
+    """x [T, C] times sigmoid(gate) (fp32), in place."""
+    x.copy_((x.float() * torch.sigmoid(gate.float())).to(x.dtype))
+
+
+# --- retention; gated gelu, squared relu, a token's side row ------------------------
+
+def _rotate_half(x, positions, inv_freq):
+    """fp32 rotation of the first 2 * len(inv_freq) entries of x [T, H, D]:
+    entry i with i + len(inv_freq), angle = float(position) * inv_freq[i]."""
+    R2 = inv_freq.numel()
+    xf = x.float()
+    ang = positions.float()[:, None, None] * inv_freq.float()
+    c, s = torch.cos(ang), torch.sin(ang)
+    u, v = xf[..., :R2], xf[..., R2:2 * R2]
+    return torch.cat([u * c - v * s, v * c + u * s, xf[..., 2 * R2:]], -1)
+
+
+def retention(q, k, v, decay, positions, inv_freq, state, state_slots, cu_seqlens, seg_start) -> torch.Tensor:
+    """Linear attention with rotary q and k over segments. q, k [T, H, D] and
+    v [T, H, V] are the raw projections; both are rotated, k is scaled by
+    D^-1/2; S_t = decay_h S_{t-1} + k_t v_t^T, o_t = S_t^T q_t. state [slots,
+    H, D, V] fp32 is read (unless seg_start == 0) and written back. Returns
+    o [T, H, V] fp32."""
+    T, H, D = q.shape
+    qf = _rotate_half(q, positions, inv_freq)
+    kf = _rotate_half(k, positions, inv_freq) * D ** -0.5
+    vf = v.float()
+    o = torch.empty(T, H, v.shape[-1], dtype=torch.float32, device=q.device)
+    cu, st, sl = cu_seqlens.tolist(), seg_start.tolist(), state_slots.tolist()
+    d = decay.float().view(H, 1, 1)
+    for b in range(len(sl)):
+        S = state[sl[b]].clone() if st[b] > 0 else torch.zeros_like(state[sl[b]])
+        for t in range(cu[b], cu[b + 1]):
+            S = d * S + kf[t].unsqueeze(-1) * vf[t].unsqueeze(-2)
+            o[t] = torch.einsum("hdv,hd->hv", S, qf[t])
+        state[sl[b]] = S
+    return o
+
+
+def gelu_glu(gate, up) -> torch.Tensor:
+    """gelu(gate) * up with the tanh-form gelu, in fp32, in gate's dtype."""
+    return (gelu_tanh(gate.float()) * up.float()).to(gate.dtype)
+
+
+def relu2(x) -> torch.Tensor:
+    """max(x, 0)^2 in fp32, in x's dtype."""
+    return x.float().clamp(min=0.0).square().to(x.dtype)
+
+
+def gelu_mul_rows(z, table, ids, col0: int) -> torch.Tensor:
+    """gelu(z [T, C]) * table[ids, col0 : col0 + C], in fp32, in z's dtype."""
+    return (gelu_tanh(z.float()) * table[ids, col0:col0 + z.shape[1]].float()).to(z.dtype)
+
+
+def add_cast(x, a, b, out_dtype) -> torch.Tensor:
+    """x (fp32, in place) += a + b (b may be None); returns x in out_dtype
+    (x itself when it is fp32)."""
+    x.add_(a.float() if b is None else a.float() + b.float())
+    return x.to(out_dtype)
 
 
 # --- layer-normed sublayers with an input convolution and a depth-weighted

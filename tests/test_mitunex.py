@@ -158,7 +158,10 @@ def run_mixer(mod, h, cuts, page=4):
 
 def load_module(mod, w, pre):
     for name, dst in mod.checkpoint_map(pre).items():
-        dst.copy_(w[name].to(dst.dtype))
+        r = 0
+        for d in dst if isinstance(dst, (list, tuple)) else [dst]:
+            d.copy_(w[name][r:r + d.shape[0]].to(d.dtype))
+            r += d.shape[0]
 
 
 def attn_module(m, width):
