@@ -59,6 +59,11 @@ def rotary_inv_freq(rot: RotarySpec) -> torch.Tensor:
     return torch.tensor(f, dtype=torch.float64).to(torch.float32)
 
 
+def single_rows(batch) -> bool:
+    """True for a step of single decoded tokens: every segment is one row."""
+    return batch.mode == "decode" or (batch.host_segs is not None and all(n == 1 for _, n in batch.host_segs))
+
+
 class FusedInput(nn.Module):
     """Several projections of the same input as ONE GEMM: the checkpoint's
     separate [out_i, in] matrices are stacked along the output dim (optionally
@@ -434,8 +439,7 @@ class LatentAttention(nn.Module):
                             batch.slot_mapping, D)
         q_abs = torch.bmm(q[:, :, :D].transpose(0, 1), self.uk)                   # [H, T, C]
         # a step of single decoded tokens: one row per workgroup, a row's keys shared out over the chip
-        single = batch.mode == "decode" or (batch.host_segs is not None
-                                            and all(n == 1 for _, n in batch.host_segs))
+        single = single_rows(batch)
         lat = ops.attn_latent_paged(q_abs.transpose(0, 1), q, st.k, batch.block_tables, batch.token_seg,
                                     batch.positions, sp.scale, sp.mask_size,
                                     s(y, "g") if sp.head_gate else None, D,
@@ -482,14 +486,29 @@ class Retention(nn.Module):
         sp = self.spec
         return LayerCacheSpec(rec=(sp.heads, sp.dim, sp.vdim))
 
+    # steps whose longest segment is shorter than this run token by token
+    MIN_CHUNK_ROWS = 16
+
+    def _chunks(self, batch):
+        """The step's rows cut into chunks for the chunk-parallel form (built
+        once per step), or None for the token-by-token form."""
+        if (batch.host_segs is None or batch.plans is None or not batch.positions.is_cuda
+                or self.spec.dim > ops.RETENTION_MAX_DIM):
+            return None
+        key = "retention_chunks"
+        if key not in batch.plans:
+            long = max((n for _, n in batch.host_segs), default=0) >= self.MIN_CHUNK_ROWS
+            batch.plans[key] = ops.retention_chunks(batch.host_segs, batch.positions.device) if long else None
+        return batch.plans[key]
+
     def forward(self, h: torch.Tensor, batch, st: LayerState) -> torch.Tensor:
         sp = self.spec
         y = self.inp(h)
         s = self.inp.split
-        o = ops.retention(s(y, "q").unflatten(1, (sp.heads, sp.dim)), s(y, "k").unflatten(1, (sp.heads, sp.dim)),
-                          s(y, "v").unflatten(1, (sp.heads, sp.vdim)), self.decay, batch.positions, self.inv_freq,
-                          st.rec, batch.state_slots, batch.cu_seqlens, batch.seg_start)
-        r = ops.gated_rmsnorm(o, None, s(y, "g"), self.eps, self.o_proj.dtype, "silu")
+        r = ops.retention_mix_out(s(y, "q").unflatten(1, (sp.heads, sp.dim)), s(y, "k").unflatten(1, (sp.heads, sp.dim)),
+                                  s(y, "v").unflatten(1, (sp.heads, sp.vdim)), s(y, "g"), self.decay, batch.positions,
+                                  self.inv_freq, st.rec, batch.state_slots, batch.cu_seqlens, batch.seg_start,
+                                  self.eps, self.o_proj.dtype, self._chunks(batch), single_rows(batch))
         return F.linear(r, self.o_proj)
 
     def checkpoint_map(self, pre: str) -> Dict[str, torch.Tensor]:

@@ -781,14 +781,49 @@ def gate_group_rmsnorm(o, weight, gate, eps, out_dtype):
     return torch_ref.gate_group_rmsnorm(o, weight, gate, eps, out_dtype)
 
 
-def retention(q, k, v, decay, positions, inv_freq, state, state_slots, cu_seqlens, seg_start):
+RETENTION_CHUNK = 64          # rows per chunk of the chunk-parallel form
+RETENTION_MAX_DIM = 128       # largest key size of the chunk-parallel form
+
+
+def retention_chunks(segs, device):
+    """Host metadata of the chunk-parallel form: segs = [(start position,
+    rows)] of a step in row order -> (chunks [NC, 4] int32: first row, rows,
+    segment, 0; seg_c0 [B + 1] int32: a segment's range of chunks)."""
+    chunks, c0, row0 = [], [0], 0
+    for b, (_, n) in enumerate(segs):
+        chunks += [(row0 + i, min(RETENTION_CHUNK, n - i), b, 0) for i in range(0, n, RETENTION_CHUNK)]
+        c0.append(len(chunks))
+        row0 += n
+    return (torch.tensor(chunks, dtype=torch.int32, device=device).reshape(-1, 4),
+            torch.tensor(c0, dtype=torch.int32, device=device))
+
+
+def retention(q, k, v, decay, positions, inv_freq, state, state_slots, cu_seqlens, seg_start, chunks=None):
     """Half-split rotation of q and k, k scaled by D^-1/2, then
-    S <- decay_h S + k v^T, o = S^T q over segments; o [T, H, V] fp32."""
+    S <- decay_h S + k v^T, o = S^T q over segments; o [T, H, V] fp32.
+    ``chunks`` (GPU, from retention_chunks): the chunk-parallel form; None:
+    token by token."""
     if _gpu(q):
         o = torch.empty((q.shape[0], q.shape[1], v.shape[2]), dtype=torch.float32, device=q.device)
-        _seq().retention(o, q, k, v, decay, positions, inv_freq, state, state_slots, cu_seqlens, seg_start)
+        e = _none(q, torch.int32)
+        ch, c0 = chunks if chunks is not None else (e, e)
+        _seq().retention(o, q, k, v, decay, positions, inv_freq, state, state_slots, cu_seqlens, seg_start, ch, c0)
         return o
     return torch_ref.retention(q, k, v, decay, positions, inv_freq, state, state_slots, cu_seqlens, seg_start)
+
+
+def retention_mix_out(q, k, v, gate, decay, positions, inv_freq, state, state_slots, cu_seqlens, seg_start, eps,
+                      out_dtype, chunks=None, single=False):
+    """retention followed by the heads' RMS norm (no weight) and silu gate
+    ([T, H*V] logits). ``single`` (GPU): every segment is one row (decode),
+    the whole of it runs as one kernel."""
+    V = v.shape[2]
+    if single and _gpu(q) and q.shape[2] <= 1024 and (V <= 256 or (V % 4 == 0 and V <= 1024)):
+        out = torch.empty((q.shape[0], q.shape[1] * V), dtype=out_dtype, device=q.device)
+        _seq().retention_step(out, q, k, v, gate, decay, positions, inv_freq, state, state_slots, seg_start, eps)
+        return out
+    o = retention(q, k, v, decay, positions, inv_freq, state, state_slots, cu_seqlens, seg_start, chunks)
+    return gated_rmsnorm(o, None, gate, eps, out_dtype, "silu")
 
 
 def gelu_glu(gate, up):

@@ -26,6 +26,12 @@ void seq_launch_add_cast(void*, float*, const void*, const void*, int64_t, int, 
 void seq_launch_retention(float*, const void*, const void*, const void*, const float*, const int64_t*, const float*,
                           float*, float*, const int*, const int*, const int*, int, int, int, int, int, int, int, int,
                           int, int, hipStream_t);
+void seq_launch_retention_chunks(float*, const void*, const void*, const void*, const float*, const int64_t*,
+                                 const float*, float*, float*, float*, const int*, const int*, const int*, const int*,
+                                 int, int, int, int, int, int, int, int, int, int, int, hipStream_t);
+void seq_launch_retention_step(void*, const void*, const void*, const void*, const void*, const float*, const int64_t*,
+                               const float*, float*, const int*, const int*, float, int, int, int, int, int, int, int,
+                               int, int, int, hipStream_t);
 void seq_launch_rmsnorm_cast(void*, const float*, const float*, int, int, float, int, hipStream_t);
 void seq_launch_sandwich_residual(float*, const void*, const void*, const float*, const float*, const float*,
                                   const float*, void*, int, int, float, int, hipStream_t);
@@ -520,25 +526,72 @@ void linear_attn_decay(torch::Tensor o, torch::Tensor q, torch::Tensor k, torch:
 }
 
 // q, k [T, H, D] and v [T, H, V] raw projections; rotation of the first 2 * inv_freq.numel() entries
+static void check_retention(const torch::Tensor& q, const torch::Tensor& k, const torch::Tensor& v,
+                            const torch::Tensor& decay, const torch::Tensor& positions, const torch::Tensor& inv_freq,
+                            const torch::Tensor& state, const torch::Tensor& slots, const torch::Tensor& seg_start) {
+  CHECK_ACT(q); CHECK_ROWS3(q); CHECK_ROWS3(k); CHECK_ROWS3(v); CHECK_SAME(k, q); CHECK_SAME(v, q);
+  CHECK_F32C(decay); CHECK_F32C(state); CHECK_I64C(positions); CHECK_F32C(inv_freq); CHECK_I32C(slots);
+  CHECK_I32C(seg_start);
+  const int T = q.size(0), H = q.size(1), D = q.size(2), V = v.size(2);
+  TORCH_CHECK(k.is_cuda() && v.is_cuda() && k.size(0) == T && v.size(0) == T && k.size(1) == H &&
+              v.size(1) == H && k.size(2) == D && positions.numel() == T && 2 * inv_freq.numel() <= D);
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == D && state.size(3) == V && decay.numel() == H);
+  TORCH_CHECK(seg_start.numel() == slots.numel());
+}
+
+// chunks empty: token by token. Else [NC, 4] int32 (first row, rows, segment, 0) and seg_c0 [B + 1]: the
+// segments' rows cut into chunks of at most 64, in order (the host built both; they are not re-read here)
 void retention(torch::Tensor o, torch::Tensor q, torch::Tensor k, torch::Tensor v, torch::Tensor decay,
                torch::Tensor positions, torch::Tensor inv_freq, torch::Tensor state, torch::Tensor slots,
-               torch::Tensor cu, torch::Tensor seg_start) {
-  CHECK_F32C(o); CHECK_ACT(q); CHECK_ROWS3(q); CHECK_ROWS3(k); CHECK_ROWS3(v); CHECK_SAME(k, q); CHECK_SAME(v, q);
-  CHECK_F32C(decay); CHECK_F32C(state); CHECK_I64C(positions); CHECK_F32C(inv_freq);
+               torch::Tensor cu, torch::Tensor seg_start, torch::Tensor chunks, torch::Tensor seg_c0) {
+  CHECK_F32C(o);
+  check_retention(q, k, v, decay, positions, inv_freq, state, slots, seg_start);
   check_segments(slots, cu, seg_start, state);
   const int T = q.size(0), H = q.size(1), D = q.size(2), V = v.size(2), B = slots.numel(), R2 = inv_freq.numel();
-  TORCH_CHECK(k.is_cuda() && v.is_cuda() && k.size(0) == T && v.size(0) == T && k.size(1) == H &&
-              v.size(1) == H && k.size(2) == D && positions.numel() == T && 2 * R2 <= D);
-  TORCH_CHECK(D <= 256, "key size above 256 is not supported by the recurrence kernel");
-  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == D && state.size(3) == V);
-  TORCH_CHECK(decay.numel() == H && o.numel() == (int64_t)T * H * V);
+  TORCH_CHECK(o.numel() == (int64_t)T * H * V);
   if (T == 0 || B == 0) return;
-  auto packed = torch::empty({(int64_t)T, (int64_t)H * (2 * D + V)}, torch::dtype(torch::kFloat).device(q.device()));
+  auto f32 = torch::dtype(torch::kFloat).device(q.device());
+  if (chunks.numel() > 0) {
+    CHECK_I32C(chunks); CHECK_I32C(seg_c0);
+    TORCH_CHECK(chunks.dim() == 2 && chunks.size(1) == 4 && seg_c0.numel() == B + 1);
+    TORCH_CHECK(D <= 128, "the chunk kernels serve key sizes up to 128");
+    const int NC = chunks.size(0);
+    auto cs = torch::empty({(int64_t)T, (int64_t)2 * R2 + 1}, f32);
+    auto U = torch::empty({(int64_t)NC, (int64_t)H, (int64_t)D, (int64_t)V}, f32);
+    seq_launch_retention_chunks(o.data_ptr<float>(), q.data_ptr(), k.data_ptr(), v.data_ptr(),
+                                decay.data_ptr<float>(), positions.data_ptr<int64_t>(), inv_freq.data_ptr<float>(),
+                                cs.data_ptr<float>(), U.data_ptr<float>(), state.data_ptr<float>(),
+                                slots.data_ptr<int>(), seg_start.data_ptr<int>(), chunks.data_ptr<int>(),
+                                seg_c0.data_ptr<int>(), T, B, NC, H, D, V, R2, (int)q.stride(0), (int)k.stride(0),
+                                (int)v.stride(0), f32flag(q), cur_stream());
+    return;
+  }
+  TORCH_CHECK(D <= 256, "key size above 256 is not supported by the recurrence kernel");
+  auto packed = torch::empty({(int64_t)T, (int64_t)H * (2 * D + V)}, f32);
   seq_launch_retention(o.data_ptr<float>(), q.data_ptr(), k.data_ptr(), v.data_ptr(), decay.data_ptr<float>(),
                        positions.data_ptr<int64_t>(), inv_freq.data_ptr<float>(), packed.data_ptr<float>(),
                        state.data_ptr<float>(), slots.data_ptr<int>(), cu.data_ptr<int>(),
                        seg_start.data_ptr<int>(), T, B, H, D, V, R2, (int)q.stride(0), (int)k.stride(0),
                        (int)v.stride(0), f32flag(q), cur_stream());
+}
+
+// one row per segment: row b continues segment b. out = silu(gate) * rms(read-out) per head, [B, H * V]
+void retention_step(torch::Tensor out, torch::Tensor q, torch::Tensor k, torch::Tensor v, torch::Tensor gate,
+                    torch::Tensor decay, torch::Tensor positions, torch::Tensor inv_freq, torch::Tensor state,
+                    torch::Tensor slots, torch::Tensor seg_start, double eps) {
+  check_retention(q, k, v, decay, positions, inv_freq, state, slots, seg_start);
+  const int B = q.size(0), H = q.size(1), D = q.size(2), V = v.size(2);
+  CHECK_ACT(out); CHECK_SAME(out, q); CHECK_ACT(gate); CHECK_SAME(gate, q); CHECK_ROWS2(gate);
+  TORCH_CHECK(slots.numel() == B, "one row per segment");
+  TORCH_CHECK(out.is_contiguous() && out.numel() == (int64_t)B * H * V && gate.size(0) == B &&
+              gate.size(1) == (int64_t)H * V);
+  TORCH_CHECK(D <= 1024 && V >= 1 && (V <= 256 || (V % 4 == 0 && V <= 1024)), "head sizes of the step kernel");
+  if (B == 0) return;
+  seq_launch_retention_step(out.data_ptr(), q.data_ptr(), k.data_ptr(), v.data_ptr(), gate.data_ptr(),
+                            decay.data_ptr<float>(), positions.data_ptr<int64_t>(), inv_freq.data_ptr<float>(),
+                            state.data_ptr<float>(), slots.data_ptr<int>(), seg_start.data_ptr<int>(), (float)eps, B,
+                            H, D, V, (int)inv_freq.numel(), (int)q.stride(0), (int)k.stride(0), (int)v.stride(0),
+                            (int)gate.stride(0), f32flag(q), cur_stream());
 }
 
 void causal_conv_silu(torch::Tensor y, torch::Tensor x, torch::Tensor w, torch::Tensor conv_state,
@@ -982,6 +1035,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gelu_mul_rows", &gelu_mul_rows);
   m.def("add_cast", &add_cast);
   m.def("retention", &retention);
+  m.def("retention_step", &retention_step);
   m.def("scale_softcap", &scale_softcap);
   m.def("scale_rows", &scale_rows);
   m.def("moe_spread_rows", &moe_spread_rows);
