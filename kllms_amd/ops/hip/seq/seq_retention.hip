@@ -77,9 +77,9 @@ __device__ __forceinline__ void ret_load_rotated(const T* __restrict__ row, cons
   }
 }
 
-// Rotated rows of one head -> LDS [RET_L][DM], zeros past n rows and D columns.
-// Column c of row r sits at c ^ (r & 31), so that both a row's and a column's
-// 32 neighbours fall on 32 banks. pw != nullptr: row r is scaled by pw[n-1-r].
+// Rotated rows of one head -> LDS [RET_L][DM + 1], zeros past n rows and D
+// columns. The odd row stride puts both a row's and a column's 32 neighbours on
+// 32 banks. pw != nullptr: row r is scaled by pw[n-1-r].
 template <typename T, int DM, int VEC>
 __device__ __forceinline__ void ret_stage(float* __restrict__ dst, const T* __restrict__ src, int64_t stride,
                                           const float* __restrict__ cs, int n, int D, int R2, float scale,
@@ -97,18 +97,18 @@ __device__ __forceinline__ void ret_stage(float* __restrict__ dst, const T* __re
       for (int e = 0; e < VEC; ++e) x[e] *= f;
     }
 #pragma unroll
-    for (int e = 0; e < VEC; ++e) dst[r * DM + ((c + e) ^ (r & 31))] = x[e];
+    for (int e = 0; e < VEC; ++e) dst[r * (DM + 1) + c + e] = x[e];
   }
 }
 
 // chunks [NC, 4] int32: first row, rows, segment, -
 // grid (NC, H): U [NC, H, D, V]
 template <typename T, int DM, int VEC>
-__global__ void __launch_bounds__(RET_THREADS) retention_chunk_u_kernel(
+__global__ void __launch_bounds__(RET_THREADS, DM > 64 ? 2 : 4) retention_chunk_u_kernel(
     float* __restrict__ U, const T* __restrict__ k, const T* __restrict__ v, const float* __restrict__ cs,
     const float* __restrict__ decay, const int* __restrict__ chunks, float kscale, int H, int D, int V, int R2,
     int k_stride, int v_stride) {
-  __shared__ float ks[RET_L * DM];
+  __shared__ float ks[RET_L * (DM + 1)];
   __shared__ float pw[RET_L + 1];
   const int c = blockIdx.x, h = blockIdx.y;
   const int row0 = chunks[4 * c], n = chunks[4 * c + 1];
@@ -122,35 +122,30 @@ __global__ void __launch_bounds__(RET_THREADS) retention_chunk_u_kernel(
   float* up = U + ((int64_t)c * H + h) * D * V;
   const T* vp = v + (int64_t)row0 * v_stride + (int64_t)h * V;
   for (int ct = wave; ct * 32 < V; ct += RET_THREADS / WAVE) {
-    const int j = ct * 32 + lr;
-    const bool on = j < V;
+    const int j = ct * 32 + lr, jc = min(j, V - 1);
     ret_f32x16 acc[DT];
 #pragma unroll
     for (int d = 0; d < DT; ++d)
 #pragma unroll
       for (int r = 0; r < 16; ++r) acc[d][r] = 0.f;
-    for (int t = 0; t < n; t += 2 * RET_KU) {
-      float b[RET_KU];
+    const float* kp = ks + half * (DM + 1) + lr;
+    for (int t = 0; t < n; t += 2 * RET_KU, kp += 2 * RET_KU * (DM + 1)) {
+      float b[RET_KU];             // rows past n: the keys there are zero
 #pragma unroll
-      for (int u = 0; u < RET_KU; ++u) {
-        const int tt = t + 2 * u + half;
-        b[u] = (on && tt < n) ? ldf(vp + (int64_t)tt * v_stride + j) : 0.f;
-      }
+      for (int u = 0; u < RET_KU; ++u) b[u] = ldf(vp + (uint32_t)(min(t + 2 * u + half, n - 1) * v_stride + jc));
 #pragma unroll
-      for (int u = 0; u < RET_KU; ++u) {
-        const int tt = t + 2 * u + half;
+      for (int u = 0; u < RET_KU; ++u)
 #pragma unroll
         for (int d = 0; d < DT; ++d)
-          acc[d] = __builtin_amdgcn_mfma_f32_32x32x2f32(ks[tt * DM + ((d * 32 + lr) ^ (tt & 31))], b[u], acc[d], 0, 0, 0);
-      }
+          acc[d] = __builtin_amdgcn_mfma_f32_32x32x2f32(kp[2 * u * (DM + 1) + d * 32], b[u], acc[d], 0, 0, 0);
     }
-    if (on) {
+    if (j < V) {
 #pragma unroll
       for (int d = 0; d < DT; ++d)
 #pragma unroll
         for (int r = 0; r < 16; ++r) {
           const int dd = d * 32 + ret_acc_row(r, half);
-          if (dd < D) up[(int64_t)dd * V + j] = acc[d][r];
+          if (dd < D) up[(uint32_t)(dd * V + j)] = acc[d][r];
         }
     }
   }
@@ -202,13 +197,14 @@ __global__ void __launch_bounds__(RET_THREADS) retention_scan_kernel(
 
 // grid (NC, H): o [T, H, V]. S0: the state before each chunk [NC, H, D, V]
 template <typename T, int DM, int VEC>
-__global__ void __launch_bounds__(RET_THREADS) retention_chunk_out_kernel(
+__global__ void __launch_bounds__(RET_THREADS, DM > 64 ? 2 : 3) retention_chunk_out_kernel(
     float* __restrict__ o, const T* __restrict__ q, const T* __restrict__ k, const T* __restrict__ v,
     const float* __restrict__ S0, const float* __restrict__ cs, const float* __restrict__ decay,
     const int* __restrict__ chunks, float kscale, int H, int D, int V, int R2, int q_stride, int k_stride,
     int v_stride) {
-  constexpr int KS = RET_L * (DM > RET_L ? DM : RET_L);      // the keys' buffer later holds the scores
-  __shared__ float qs[RET_L * DM];
+  constexpr int QS = DM + 1, PS = RET_L + 1;                 // row strides of the staged rows and of the scores
+  constexpr int KS = RET_L * (QS > PS ? QS : PS);            // the keys' buffer later holds the scores
+  __shared__ float qs[RET_L * QS];
   __shared__ float ks[KS];
   __shared__ float pw[RET_L + 1];
   const int c = blockIdx.x, h = blockIdx.y;
@@ -221,52 +217,46 @@ __global__ void __launch_bounds__(RET_THREADS) retention_chunk_out_kernel(
   __syncthreads();
   // scores q_i . k_j, one 32 x 32 tile per wave (the tile above the diagonal is never read)
   const int it = wave >> 1, jt = wave & 1;
-  const bool tile = it >= jt && it * 32 < n;
+  const bool tile = it >= jt;
   ret_f32x16 s;
 #pragma unroll
   for (int r = 0; r < 16; ++r) s[r] = 0.f;
   if (tile) {
-    const float* qr = qs + (it * 32 + lr) * DM;
-    const float* kr = ks + (jt * 32 + lr) * DM;
-#pragma unroll
-    for (int d = 0; d < DM; d += 2)
-      s = __builtin_amdgcn_mfma_f32_32x32x2f32(qr[(d + half) ^ lr], kr[(d + half) ^ lr], s, 0, 0, 0);
+    const float* qr = qs + (it * 32 + lr) * QS + half;
+    const float* kr = ks + (jt * 32 + lr) * QS + half;
+#pragma unroll 16
+    for (int d = 0; d < DM; d += 2) s = __builtin_amdgcn_mfma_f32_32x32x2f32(qr[d], kr[d], s, 0, 0, 0);
   }
   __syncthreads();
-  float* ps = ks;                              // [RET_L][RET_L], column j of row i at j ^ (i & 31)
+  float* ps = ks;                              // [RET_L][PS]
   if (tile) {
 #pragma unroll
     for (int r = 0; r < 16; ++r) {
       const int i = it * 32 + ret_acc_row(r, half), j = jt * 32 + lr;
-      ps[i * RET_L + (j ^ (i & 31))] = i >= j ? s[r] * pw[i - j] : 0.f;
+      ps[i * PS + j] = i >= j ? s[r] * pw[i - j] : 0.f;
     }
   }
   __syncthreads();
   const float* sp = S0 + ((int64_t)c * H + h) * D * V;
   const T* vp = v + (int64_t)row0 * v_stride + (int64_t)h * V;
-  const float* q0 = qs + lr * DM;
-  const float* q1 = qs + (32 + lr) * DM;
-  const float* p0 = ps + lr * RET_L;
-  const float* p1 = ps + (32 + lr) * RET_L;
-  // rows past n are computed with the others and not stored
+  float* op = o + ((int64_t)row0 * H + h) * V;
+  const int HV = H * V;
+  // rows past n, columns past V and entries past D are computed with the others (their staged queries or
+  // scores are zero, so what the clamped loads bring does not matter) and not stored
   for (int ct = wave; ct * 32 < V; ct += RET_THREADS / WAVE) {
-    const int j = ct * 32 + lr;
-    const bool on = j < V;
+    const int j = ct * 32 + lr, jc = min(j, V - 1);
     ret_f32x16 a0, a1;
 #pragma unroll
     for (int r = 0; r < 16; ++r) { a0[r] = 0.f; a1[r] = 0.f; }
-    for (int d = 0; d < D; d += 2 * RET_KU) {
+    const float* qp = qs + lr * QS + half;
+    for (int d = 0; d < D; d += 2 * RET_KU, qp += 2 * RET_KU) {
       float b[RET_KU];
 #pragma unroll
-      for (int u = 0; u < RET_KU; ++u) {
-        const int dd = d + 2 * u + half;
-        b[u] = (on && dd < D) ? sp[(int64_t)dd * V + j] : 0.f;
-      }
+      for (int u = 0; u < RET_KU; ++u) b[u] = sp[(uint32_t)(min(d + 2 * u + half, D - 1) * V + jc)];
 #pragma unroll
       for (int u = 0; u < RET_KU; ++u) {
-        const int dd = d + 2 * u + half;
-        a0 = __builtin_amdgcn_mfma_f32_32x32x2f32(q0[dd ^ lr], b[u], a0, 0, 0, 0);
-        a1 = __builtin_amdgcn_mfma_f32_32x32x2f32(q1[dd ^ lr], b[u], a1, 0, 0, 0);
+        a0 = __builtin_amdgcn_mfma_f32_32x32x2f32(qp[2 * u], b[u], a0, 0, 0, 0);
+        a1 = __builtin_amdgcn_mfma_f32_32x32x2f32(qp[2 * u + 32 * QS], b[u], a1, 0, 0, 0);
       }
     }
 #pragma unroll
@@ -275,28 +265,25 @@ __global__ void __launch_bounds__(RET_THREADS) retention_chunk_out_kernel(
       a0[r] *= pw[i + 1];
       a1[r] *= pw[i + 33];
     }
-    for (int t = 0; t < n; t += 2 * RET_KU) {
+    const float* pp = ps + lr * PS + half;
+    for (int t = 0; t < n; t += 2 * RET_KU, pp += 2 * RET_KU) {
       float b[RET_KU];
 #pragma unroll
-      for (int u = 0; u < RET_KU; ++u) {
-        const int tt = t + 2 * u + half;
-        b[u] = (on && tt < n) ? ldf(vp + (int64_t)tt * v_stride + j) : 0.f;
-      }
+      for (int u = 0; u < RET_KU; ++u) b[u] = ldf(vp + (uint32_t)(min(t + 2 * u + half, n - 1) * v_stride + jc));
       if (t < 32) {                            // tokens 32.. lie after rows 0..31
 #pragma unroll
-        for (int u = 0; u < RET_KU; ++u)
-          a0 = __builtin_amdgcn_mfma_f32_32x32x2f32(p0[(t + 2 * u + half) ^ lr], b[u], a0, 0, 0, 0);
+        for (int u = 0; u < RET_KU; ++u) a0 = __builtin_amdgcn_mfma_f32_32x32x2f32(pp[2 * u], b[u], a0, 0, 0, 0);
       }
 #pragma unroll
       for (int u = 0; u < RET_KU; ++u)
-        a1 = __builtin_amdgcn_mfma_f32_32x32x2f32(p1[(t + 2 * u + half) ^ lr], b[u], a1, 0, 0, 0);
+        a1 = __builtin_amdgcn_mfma_f32_32x32x2f32(pp[2 * u + 32 * PS], b[u], a1, 0, 0, 0);
     }
-    if (on) {
+    if (j < V) {
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
         const int i = ret_acc_row(r, half);
-        if (i < n) o[((int64_t)(row0 + i) * H + h) * V + j] = a0[r];
-        if (i + 32 < n) o[((int64_t)(row0 + i + 32) * H + h) * V + j] = a1[r];
+        if (i < n) op[(uint32_t)(i * HV + j)] = a0[r];
+        if (i + 32 < n) op[(uint32_t)((i + 32) * HV + j)] = a1[r];
       }
     }
   }
