@@ -124,7 +124,7 @@ class BavesunForCausalLM(ListedLayerLM):
                              batch.state_slots, batch.cu_seqlens, batch.seg_start, batch.token_seg)
         # the norm weight of whatever reads the stream after each layer run
         scales = [self.layers[i].norm1.scale for i in self.runs] + [self.final_norm.scale]
-        h = ops.rmsnorm_cast(x, scales[0], eps, self.dtype)
+        h, _ = ops.group_norm_pair(x, None, None, scales[0], None, 1, eps, self.dtype)
         for run, i in enumerate(self.runs):
             layer = self.layers[i]
             a = layer.mix(h, batch, states[run])
