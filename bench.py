@@ -419,6 +419,8 @@ def main():
         coord = sched.coordinator
         sched.shutdown()      # join the worker thread first …
         coord.stop()          # … then release the followers
+    elif getattr(eng_client, "_scheduler", None) is not None:
+        eng_client._scheduler.shutdown()   # no worker thread is left running torch code at interpreter exit
     if dist is not None:
         dist.barrier()
         dist.destroy_process_group()
