@@ -156,11 +156,13 @@ class MlstmSpec(BaseModel):
 
 class SharedExpertSpec(BaseModel):
     """An expert that every token passes; its output is scaled by sigmoid of
-    one more projection of the input (a scalar per token). ``limit`` is the
-    clamp of a clamped-GLU expert (None: as the routed experts' form says)."""
+    one more projection of the input (a scalar per token), or added as it is
+    (``gated`` False). ``limit`` is the clamp of a clamped-GLU expert (None:
+    as the routed experts' form says)."""
 
     ff: int
     limit: Optional[float] = None
+    gated: bool = True
 
 
 class RoutedExpertsSpec(BaseModel):
@@ -172,8 +174,9 @@ class RoutedExpertsSpec(BaseModel):
     choice is made on score (+ correction, if the checkpoint has one) among
     the experts of the best ``group_keep`` of ``group_count`` groups of
     neighbours. The chosen scores weigh the experts, renormalised to sum 1 or
-    as they are; the weight multiplies the expert's output or its input
-    (``weight_on``). ``shared``: one more expert that runs for every token."""
+    as they are, times ``scale``; the weight multiplies the expert's output or
+    its input (``weight_on``). ``shared``: one more expert that runs for every
+    token."""
 
     kind: Literal["moe"] = "moe"
     experts: int
@@ -184,6 +187,7 @@ class RoutedExpertsSpec(BaseModel):
     ff: int
     score: Literal["softmax", "sigmoid", "top_softmax"] = "softmax"
     renormalize: bool = True
+    scale: float = 1.0
     correction: bool = True
     weight_on: Literal["output", "input"] = "output"
     shared: Optional[SharedExpertSpec] = None
@@ -337,7 +341,8 @@ def _medilix_preset(vocab, width, depth, heads, kv_heads, dim, mask, keep, r_hea
 class LatentAttnSpec(BaseModel):
     """Softmax attention whose keys and values are up-projections of one
     shared latent row per token. Per head the query has ``dim`` unrotated and
-    ``rot_dim`` rotated entries; the token's down-projection gives the latent
+    ``rot_dim`` rotated entries; with ``q_rank`` > 0 the queries are
+    up-projections of an RMS-normed latent of their own. The token's down-projection gives the latent
     (``kv_rank`` entries, RMS-normed) and one rotated key part shared by all
     heads. Only those two are cached. Causal sliding window of ``mask_size``
     positions (0 = plain causal). Output gate: sigmoid of one logit per head
@@ -350,6 +355,7 @@ class LatentAttnSpec(BaseModel):
     rot_dim: int
     vdim: int
     kv_rank: int
+    q_rank: int = 0
     scale: float
     mask_size: int = 0
     rot: RotarySpec = Field(default_factory=RotarySpec)
@@ -360,11 +366,11 @@ class LatentAttnSpec(BaseModel):
 
 class ActFFSpec(BaseModel):
     """Feed-forward W_down act(W_up h), or W_down (act(W_gate h) * (W_up h)) if
-    ``gated``; act = tanh-form gelu."""
+    ``gated``; act = tanh-form gelu, or max(z, 0)^2 ("relu2", ungated)."""
 
     kind: Literal["dense"] = "dense"
     ff: int
-    act: Literal["gelu_tanh"] = "gelu_tanh"
+    act: Literal["gelu_tanh", "relu2"] = "gelu_tanh"
     gated: bool = False
 
 
@@ -740,6 +746,130 @@ def _bavesun_preset(vocab, width, depth, r_heads, r_dim, r_vdim, heads, dim, rot
                              layers=layers, loop=LoopSpec(**loop) if loop else None)
 
 
+class DiffAttnSpec(BaseModel):
+    """Differential attention: two softmax maps per head over the same values,
+    combined as (map 1 - lambda map 2), lambda = exp(lq1.lk1) - exp(lq2.lk2) +
+    ``diff`` (one number per layer), then RMS-normed per head (no weight) and
+    scaled by 1 - diff. ``dim`` is the query / key size of one map. Plain
+    causal, grouped heads, no rotation; the projections have biases and pass a
+    short causal convolution of ``conv`` taps; queries are scaled by
+    1 + temp_coef ln(floor((p + 1) / temp_every) + 1) at position p.
+    ``kv_from``: the layer projects queries only and reads the keys and values
+    of that earlier layer."""
+
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    diff: float
+    conv: int = 1
+    temp_coef: float = 0.0
+    temp_every: int = 1
+    kv_from: Optional[int] = None
+
+
+class DimuvikLayerSpec(BaseModel):
+    type: Literal["attention", "latent_attention"]
+    attention: Optional[DiffAttnSpec] = None
+    latent: Optional[LatentAttnSpec] = None
+    mlp: Optional[Union[ActFFSpec, RoutedExpertsSpec]] = None
+
+
+class DimuvikArchConfig(BaseModel):
+    """A decoder whose sublayers are normed before and after by dynamic tanh,
+    x <- x + dyt(sublayer(dyt(x))), dyt(v) = tanh(alpha v) w + b. Mixers:
+    differential attention (optionally on an earlier layer's cache), or latent
+    attention with a query latent and a sink; feed-forward: squared relu,
+    routed silu experts with a shared expert, or none. The LM head is a matrix
+    of its own. Every size comes from the checkpoint's config.json."""
+
+    arch: Literal["dimuvik"] = "dimuvik"
+    vocab_size: int
+    hidden_size: int
+    rms_norm_eps: float = 1e-6          # of the norms inside the mixers
+    embed_scale: float = 1.0
+    layers: List[DimuvikLayerSpec]
+    max_position_embeddings: int = 1 << 24
+    tie_word_embeddings: bool = False
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @classmethod
+    def from_checkpoint_config(cls, d: dict, shapes: Optional[dict] = None) -> "DimuvikArchConfig":
+        """Parse the family's config.json (keys: vocab, width, norm.eps,
+        embedding.scale, layers[].type / .mixer / .mlp)."""
+        layers = []
+        for li, spec in enumerate(d["layers"]):
+            m, mlp, kind = spec["mixer"], spec.get("mlp"), spec["type"]
+            ff = None
+            if mlp:
+                if mlp["kind"] == "dense":
+                    ff = ActFFSpec(ff=mlp["ff"], act="relu2")
+                elif mlp["kind"] == "moe":
+                    r, sh = mlp["router"], mlp.get("shared")
+                    ff = RoutedExpertsSpec(experts=r["experts"], top=r["top"], ff=mlp["expert"]["ff"], score="softmax",
+                                           renormalize=False, scale=r.get("scale", 1.0), correction=True,
+                                           shared=SharedExpertSpec(ff=sh["ff"], gated=False) if sh else None)
+                else:
+                    raise ValueError(f"unknown feed-forward kind {mlp['kind']!r}")
+            if kind == "attention":
+                src, temp = m.get("kv_from"), m.get("q_temp") or {}
+                if src is not None:
+                    other = d["layers"][src] if 0 <= src < li else None
+                    if other is None or other["type"] != "attention" or other["mixer"].get("kv_from") is not None:
+                        raise ValueError(f"layer {li}: kv_from {src} does not name an earlier attention layer "
+                                         f"with keys and values of its own")
+                    if any(other["mixer"][n] != m[n] for n in ("kv_heads", "dim", "vdim")):
+                        raise ValueError(f"layer {li}: the keys and values of layer {src} have other sizes")
+                layers.append(DimuvikLayerSpec(type=kind, mlp=ff, attention=DiffAttnSpec(
+                    heads=m["heads"], kv_heads=m["kv_heads"], dim=m["dim"], vdim=m["vdim"], scale=m["scale"],
+                    diff=m["diff"], conv=m.get("conv") or 1, temp_coef=temp.get("coef") or 0.0,
+                    temp_every=temp.get("every") or 1, kv_from=src)))
+            elif kind == "latent_attention":
+                rot = m.get("rot") or {}
+                if rot.get("dims", m["rot_dim"]) != m["rot_dim"]:
+                    raise ValueError("the rotated part of a latent-attention head is rotated whole")
+                layers.append(DimuvikLayerSpec(type=kind, mlp=ff, latent=LatentAttnSpec(
+                    heads=m["heads"], dim=m["dim"], rot_dim=m["rot_dim"], vdim=m["vdim"], kv_rank=m["kv_rank"],
+                    q_rank=m["q_rank"], scale=m["scale"],
+                    rot=RotarySpec(base=rot.get("base", 10000.0), dims=m["rot_dim"]), head_gate=False, sink=True)))
+            else:
+                raise ValueError(f"unknown layer type {kind!r}")
+        return cls(vocab_size=d["vocab"], hidden_size=d["width"], rms_norm_eps=d["norm"]["eps"],
+                   embed_scale=(d.get("embedding") or {}).get("scale", 1.0), layers=layers)
+
+
+def _dimuvik_preset(vocab, width, depth, a_heads, a_kv, a_dim, a_vdim, heads, dim, rot_dim, vdim, kv_rank, q_rank, ff,
+                    experts, top, expert_ff, shared_ff, pattern="LaAl") -> DimuvikArchConfig:
+    """Random-init presets of the family: ``pattern`` repeats over the depth
+    ('a' differential attention, 'l' latent attention; upper case: dense
+    feed-forward, lower case: routed experts). Of two neighbouring attention
+    layers the second reads the first one's keys and values."""
+    import math as _math
+
+    layers: List[DimuvikLayerSpec] = []
+    for i in range(depth):
+        c = pattern[i % len(pattern)]
+        mlp = (ActFFSpec(ff=ff, act="relu2") if c.isupper() else
+               RoutedExpertsSpec(experts=experts, top=top, ff=expert_ff, score="softmax", renormalize=False, scale=2.0,
+                                 shared=SharedExpertSpec(ff=shared_ff, gated=False) if shared_ff else None))
+        if c in "aA":
+            prev = layers[-1].attention if layers else None
+            layers.append(DimuvikLayerSpec(type="attention", mlp=mlp, attention=DiffAttnSpec(
+                heads=a_heads, kv_heads=a_kv, dim=a_dim, vdim=a_vdim, scale=1.0 / _math.sqrt(a_dim),
+                diff=0.8 - 0.6 * _math.exp(-0.3 * i), conv=4, temp_coef=0.1, temp_every=1024,
+                kv_from=i - 1 if prev is not None and prev.kv_from is None else None)))
+        else:
+            layers.append(DimuvikLayerSpec(type="latent_attention", mlp=mlp, latent=LatentAttnSpec(
+                heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, kv_rank=kv_rank, q_rank=q_rank,
+                scale=1.0 / _math.sqrt(dim + rot_dim), rot=RotarySpec(base=1e6, dims=rot_dim),
+                head_gate=False, sink=True)))
+    return DimuvikArchConfig(vocab_size=vocab, hidden_size=width, embed_scale=_math.sqrt(width), layers=layers)
+
+
 class HybridLayerSpec(BaseModel):
     type: Literal["parallel", "channel_delta"]
     parallel: Optional[ParallelMixerSpec] = None
@@ -987,6 +1117,24 @@ MODEL_PRESETS: dict = {
     "bavesun-1b-l6": _bavesun_preset(
         vocab=32000, width=2048, depth=6, r_heads=16, r_dim=64, r_vdim=128, heads=16, dim=128, rot_dim=64,
         vdim=128, kv_rank=512, ff=8192, experts=8, top=2, expert_ff=6144, side_dim=128, pattern="Rl"),
+    # Dimuvik family (dynamic-tanh norms before and after every sublayer;
+    # differential attention, in pairs that share keys and values, and latent
+    # attention with a query latent and a sink; squared relu and routed experts)
+    "tiny-dimuvik": _dimuvik_preset(
+        vocab=512, width=64, depth=4, a_heads=4, a_kv=2, a_dim=8, a_vdim=24, heads=4, dim=16, rot_dim=8, vdim=24,
+        kv_rank=32, q_rank=24, ff=96, experts=6, top=2, expert_ff=48, shared_ff=40),
+    "mid-dimuvik": _dimuvik_preset(
+        vocab=2048, width=512, depth=4, a_heads=4, a_kv=2, a_dim=64, a_vdim=128, heads=8, dim=64, rot_dim=32, vdim=64,
+        kv_rank=128, q_rank=192, ff=1024, experts=8, top=2, expert_ff=256, shared_ff=256),
+    # layer shapes of real models at reduced depth, beside llama-/mitunex-{1b,8b}-l6
+    "dimuvik-8b-l6": _dimuvik_preset(
+        vocab=32000, width=4096, depth=6, a_heads=16, a_kv=4, a_dim=128, a_vdim=256, heads=32, dim=128, rot_dim=64,
+        vdim=128, kv_rank=512, q_rank=1536, ff=14336, experts=8, top=2, expert_ff=7168, shared_ff=2048,
+        pattern="LaAlAa"),
+    "dimuvik-1b-l6": _dimuvik_preset(
+        vocab=32000, width=2048, depth=6, a_heads=8, a_kv=2, a_dim=128, a_vdim=256, heads=16, dim=128, rot_dim=64,
+        vdim=128, kv_rank=512, q_rank=768, ff=8192, experts=8, top=2, expert_ff=4096, shared_ff=1024,
+        pattern="LaAlAa"),
 }
 
 
@@ -1089,12 +1237,12 @@ class EngineConfig(BaseModel):
         with open(cfg_path) as f:
             hf = json.load(f)
         family = str(hf.get("architecture", "")).lower()
-        if family in ("zutalix", "medilix", "mitunex", "pironex", "bavesun"):
+        if family in ("zutalix", "medilix", "mitunex", "pironex", "bavesun", "dimuvik"):
             from .weights import safetensors_shapes
 
             reader = {"zutalix": HybridArchConfig, "medilix": MedilixArchConfig,
                       "mitunex": MitunexArchConfig, "pironex": PironexArchConfig,
-                      "bavesun": BavesunArchConfig}[family]
+                      "bavesun": BavesunArchConfig, "dimuvik": DimuvikArchConfig}[family]
             return reader.from_checkpoint_config(hf, safetensors_shapes(os.path.dirname(cfg_path)))
         arch = "mixtral" if "mixtral" in hf.get("model_type", "").lower() or hf.get("num_local_experts") else "llama"
         return ModelArchConfig(

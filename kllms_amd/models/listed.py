@@ -40,6 +40,8 @@ class ListedLayerLM(nn.Module):
                 raise RuntimeError(f"checkpoint tensor {name!r} has no place in this model")
             # a list: the checkpoint tensor's rows are dealt to several parameter slices in turn
             parts = dst if isinstance(dst, (list, tuple)) else [dst]
+            if t.dim() == 0:                 # a stored scalar fills a one-element parameter
+                t = t.reshape(1)
             shape = (sum(d.shape[0] for d in parts),) + tuple(parts[0].shape[1:])
             if shape != tuple(t.shape) or any(tuple(d.shape[1:]) != shape[1:] for d in parts):
                 raise RuntimeError(f"{name}: checkpoint shape {tuple(t.shape)} != model {shape}")

@@ -4,7 +4,7 @@ linear attention, the gated delta rule with per-channel decay and short
 convolutions, the clamped GLU; windowed attention with kept first tokens and
 a sink, the wkv and mlstm recurrences, routed experts; latent attention and
 the gelu feed-forwards; retention, the zero-centred norm weight and the token
-side input. Each runs on "segment" batches
+side input; differential attention and the dynamic-tanh norm. Each runs on "segment" batches
 (ForwardBatch.seg_start / state_slots / token_seg): any mix of prompt
 portions and single decoded tokens, attention keys found through the block
 table and recurrent state carried in per-sequence slots.
@@ -25,8 +25,8 @@ import torch.nn as nn
 import torch.nn.functional as F
 
 from .. import ops
-from ..engine.config import (ActFFSpec, BlockAttnSpec, ChannelDeltaSpec, DecayLinearAttnSpec, GluSpec,
-                             LatentAttnSpec, Mamba2Spec, MaskedAttnSpec, MlstmSpec, ParallelMixerSpec,
+from ..engine.config import (ActFFSpec, BlockAttnSpec, ChannelDeltaSpec, DecayLinearAttnSpec, DiffAttnSpec,
+                             GluSpec, LatentAttnSpec, Mamba2Spec, MaskedAttnSpec, MlstmSpec, ParallelMixerSpec,
                              PoolWindowAttnSpec, RetentionSpec, RotarySpec, RoutedExpertsSpec, WkvSpec)
 from ..engine.kvcache import LayerCacheSpec, LayerState
 
@@ -399,7 +399,8 @@ class LatentAttention(nn.Module):
         out     = W_uv sum_j p_j c_j
     and the attention proper runs in the latent space for all heads against
     the same cached rows: W_uk is applied to the queries before it (one
-    batched product over the heads) and W_uv to its result. Sliding causal
+    batched product over the heads) and W_uv to its result. With a q_rank the
+    queries are W_uq (rms(W_dq h) w). Sliding causal
     window or plain causal, optional sink (a learned number per head in the
     softmax denominator), sigmoid output gate per head, per element of the
     concatenated heads, or none; q, the down-projection and the gate share one
@@ -412,11 +413,14 @@ class LatentAttention(nn.Module):
         self.spec = spec
         self.eps = eps
         H, D, R, V, C = spec.heads, spec.dim, spec.rot_dim, spec.vdim, spec.kv_rank
-        parts = [("q", H * (D + R)), ("dkv", C + R)]
+        Q = spec.q_rank
+        parts = [("dq", Q) if Q else ("q", H * (D + R)), ("dkv", C + R)]
         assert not (spec.head_gate and spec.elem_gate)
         if spec.head_gate or spec.elem_gate:
             parts.append(("g", H if spec.head_gate else H * V))
         self.inp = FusedInput(hidden, parts, dtype)
+        self.dq_norm = _param(Q, dtype=torch.float32) if Q else None
+        self.uq = _param(H * (D + R), Q, dtype=dtype) if Q else None
         self.dkv_norm = _param(C, dtype=torch.float32)
         self.uk = _param(H, D, C, dtype=dtype)
         self.uv = _param(H, C, V, dtype=dtype)
@@ -434,7 +438,8 @@ class LatentAttention(nn.Module):
         H, D, R, V = sp.heads, sp.dim, sp.rot_dim, sp.vdim
         y = self.inp(h)
         s = self.inp.split
-        q = s(y, "q").unflatten(1, (H, D + R))
+        q = s(y, "q") if self.uq is None else F.linear(ops.rmsnorm_rows(s(y, "dq"), self.dq_norm, self.eps), self.uq)
+        q = q.unflatten(1, (H, D + R))
         ops.latent_kv_store(q, s(y, "dkv"), self.dkv_norm, self.eps, batch.positions, self.inv_freq, st.k,
                             batch.slot_mapping, D)
         q_abs = torch.bmm(q[:, :, :D].transpose(0, 1), self.uk)                   # [H, T, C]
@@ -452,6 +457,8 @@ class LatentAttention(nn.Module):
 
     def checkpoint_map(self, pre: str) -> Dict[str, torch.Tensor]:
         m = {pre + n: self.inp.slot(n) for n in self.inp.parts}
+        if self.uq is not None:
+            m[pre + "dq.norm"], m[pre + "uq"] = self.dq_norm, self.uq
         m[pre + "dkv.norm"] = self.dkv_norm
         m[pre + "uk"] = self.uk.view(-1, self.spec.kv_rank)
         m[pre + "uv"] = [head.t() for head in self.uv]      # the checkpoint's rows, V per head
@@ -633,6 +640,99 @@ class PoolWindowAttention(nn.Module):
         return m
 
 
+class DynamicTanh(nn.Module):
+    """Norm that computes no statistics: tanh(alpha v) w + b with one number
+    alpha. The kernels take the three as they are (``args``)."""
+
+    def __init__(self, width: int):
+        super().__init__()
+        self.alpha = _param(1, dtype=torch.float32)
+        self.weight = _param(width, dtype=torch.float32)
+        self.bias = _param(width, dtype=torch.float32)
+
+    @property
+    def args(self) -> Tuple[torch.Tensor, torch.Tensor, torch.Tensor]:
+        return self.alpha, self.weight, self.bias
+
+    def checkpoint_map(self, name: str) -> Dict[str, torch.Tensor]:
+        return {name: self.weight, name + ".b": self.bias, name + ".alpha": self.alpha}
+
+
+class DiffAttention(nn.Module):
+    """Differential attention over the paged cache. Every query and key head
+    holds two maps of ``dim`` entries over the same values; with a_1, a_2 the
+    maps' outputs and lambda = exp(lq1 . lk1) - exp(lq2 . lk2) + diff,
+        o = rms(a_1 - lambda a_2) (1 - diff)
+    per head. q, k and v (with biases) share one input GEMM and pass a short
+    causal convolution, whose inputs are carried in the slot; queries take the
+    position-dependent temperature. A layer with ``kv_from`` projects queries
+    only and reads the keys and values another layer cached in this step."""
+
+    LAMBDAS = ("lq1", "lk1", "lq2", "lk2")
+
+    def __init__(self, spec: DiffAttnSpec, hidden: int, eps: float, dtype):
+        super().__init__()
+        assert spec.heads % spec.kv_heads == 0 and spec.conv >= 1
+        self.spec = spec
+        self.eps = eps
+        self.own_kv = spec.kv_from is None
+        parts = [("q", spec.heads * 2 * spec.dim)]
+        if self.own_kv:
+            parts += [("k", spec.kv_heads * 2 * spec.dim), ("v", spec.kv_heads * spec.vdim)]
+        self.inp = FusedInput(hidden, parts, dtype, bias_parts=[n for n, _ in parts])
+        # taps-major over the fused projection's columns as laid out (zero taps in alignment gaps)
+        self.conv = nn.Parameter(torch.zeros(spec.conv, self.inp.weight.shape[0], dtype=torch.float32),
+                                 requires_grad=False)
+        self.lambdas = _param(4, spec.dim, dtype=torch.float32)
+        self.lam = 0.0
+        self.o_proj = _param(hidden, spec.heads * spec.vdim, dtype=dtype)
+
+    def fold(self) -> None:
+        """The layer's lambda, once its vectors are in place."""
+        lq1, lk1, lq2, lk2 = self.lambdas.double().cpu()
+        self.lam = math.exp(float(lq1 @ lk1)) - math.exp(float(lq2 @ lk2)) + self.spec.diff
+
+    def cache_spec(self) -> LayerCacheSpec:
+        sp = self.spec
+        return LayerCacheSpec(kv=(sp.kv_heads, 2 * sp.dim, sp.vdim) if self.own_kv else None, kv_of=sp.kv_from,
+                              conv=(self.conv.shape[1], sp.conv - 1))
+
+    def _tiles(self, batch):
+        """The step's rows as query tiles and single rows (built once per
+        step), None for a step of single decoded tokens."""
+        if single_rows(batch):
+            return None
+        assert batch.host_segs is not None, "a step with prompt portions is built on the host"
+        if batch.plans is None:
+            batch.plans = {}
+        rows = ops.diff_tile_rows(self.spec.heads, self.spec.kv_heads)
+        key = ("diff_tiles", rows)
+        if key not in batch.plans:
+            batch.plans[key] = ops.diff_tiles(batch.host_segs, rows, batch.positions.device)
+        return batch.plans[key]
+
+    def forward(self, h: torch.Tensor, batch, st: LayerState) -> torch.Tensor:
+        sp = self.spec
+        T = h.shape[0]
+        p = self.inp.parts
+        q = ops.conv_qkv_store(self.inp(h), self.conv, st.conv, batch.state_slots, batch.cu_seqlens, batch.seg_start,
+                               batch.token_seg, batch.positions, p["q"], sp.temp_coef, sp.temp_every, p.get("k"),
+                               p.get("v"), st.k, st.v, batch.slot_mapping, single_rows(batch))
+        att = ops.attn_diff_paged(q.view(T, sp.heads, 2 * sp.dim), st.k, st.v, batch.block_tables, batch.token_seg,
+                                  batch.positions, sp.scale, self.lam, 1.0 - sp.diff, self.eps, self._tiles(batch))
+        return F.linear(att.view(T, -1), self.o_proj)
+
+    def checkpoint_map(self, pre: str) -> Dict[str, torch.Tensor]:
+        m = {}
+        for n, (off, size) in self.inp.parts.items():
+            m[pre + n], m[pre + n + ".b"] = self.inp.slot(n), self.inp.bias_slot(n)
+            m[pre + n + ".conv"] = self.conv.t()[off:off + size]
+        for i, n in enumerate(self.LAMBDAS):
+            m[pre + n] = self.lambdas[i]
+        m[pre + "o"] = self.o_proj
+        return m
+
+
 class Mamba2Mixer(nn.Module):
     """State-space mixer. One input GEMM gives [z | x | B | C | dt]; x, B, C
     pass a short causal convolution (with bias) and silu together; per head h
@@ -689,10 +789,12 @@ class Mamba2Mixer(nn.Module):
 
 class ActFF(nn.Module):
     """y = W_down act(W_up h), or W_down (act(W_gate h) * (W_up h)) when gated
-    (gate and up share one GEMM), with the tanh-form gelu."""
+    (gate and up share one GEMM), with the tanh-form gelu or (ungated) the
+    squared relu."""
 
     def __init__(self, spec: ActFFSpec, hidden: int, dtype):
         super().__init__()
+        assert spec.act == "gelu_tanh" or not spec.gated
         self.spec = spec
         self.inp = FusedInput(hidden, [("gate", spec.ff), ("up", spec.ff)], dtype) if spec.gated else None
         self.up = None if spec.gated else _param(spec.ff, hidden, dtype=dtype)
@@ -702,7 +804,8 @@ class ActFF(nn.Module):
         if self.inp is not None:
             y = self.inp(h)
             return F.linear(ops.gelu_glu(self.inp.split(y, "gate"), self.inp.split(y, "up")), self.down)
-        return F.linear(ops.gelu_tanh(F.linear(h, self.up)), self.down)
+        act = ops.relu2 if self.spec.act == "relu2" else ops.gelu_tanh
+        return F.linear(act(F.linear(h, self.up)), self.down)
 
     def checkpoint_map(self, pre: str) -> Dict[str, torch.Tensor]:
         if self.inp is not None:
@@ -823,11 +926,11 @@ class RoutedExperts(nn.Module):
     squared-relu experts. The router runs in fp32: scores are the softmax over
     all outputs, the sigmoid of each, or the softmax over the chosen logits;
     the choice is made on score (+ correction) within the best groups of neighbouring experts; the
-    chosen scores, renormalised or as they are, weigh the experts — their
+    chosen scores, renormalised or as they are, times a constant, weigh the experts — their
     outputs, or (``weight_on = "input"``) their inputs: expert(w h). The last
     ``identity`` router outputs stand for experts that return their input and
     have no weights. An optional shared expert runs for every row and is
-    added times sigmoid of one more projection of the row.
+    added, times sigmoid of one more projection of the row if it is gated.
 
     Few rows (decode): every expert runs on every row as two batched GEMMs
     (the weights stream from memory once either way, and shapes do not depend
@@ -863,7 +966,8 @@ class RoutedExperts(nn.Module):
         self.shared_inp = self.shared_down = None
         if spec.shared is not None:
             sff = spec.shared.ff
-            self.shared_inp = FusedInput(hidden, [("gate", sff), ("up", sff), ("sg", 1)], dtype)
+            self.shared_inp = FusedInput(hidden, [("gate", sff), ("up", sff)] +
+                                         ([("sg", 1)] if spec.shared.gated else []), dtype)
             self.shared_down = _param(hidden, sff, dtype=dtype)
 
     def _act(self, gate: torch.Tensor, up: torch.Tensor, limit: Optional[float] = None) -> torch.Tensor:
@@ -885,7 +989,7 @@ class RoutedExperts(nn.Module):
         on_input = sp.weight_on == "input"
         dense = T <= self.DENSE_MAX_ROWS and E * T <= self.DENSE_MAX_PAIRS
         idx, w, rowidx = ops.moe_route_rows(h, self.router, self.correction, top, sp.group_count, sp.group_keep,
-                                            E, dense, sp.score, sp.renormalize)
+                                            E, dense, sp.score, sp.renormalize, sp.scale)
         if dense:
             if on_input:
                 # expert e reads w[t, e] h[t] where it was chosen (zero rows elsewhere; they are never read back)
@@ -918,7 +1022,7 @@ class RoutedExperts(nn.Module):
             ys = self.shared_inp(h)
             ss = self.shared_inp.split
             extra = F.linear(self._act(ss(ys, "gate"), ss(ys, "up"), sp.shared.limit), self.shared_down)
-            gate = ss(ys, "sg")[:, 0]
+            gate = ss(ys, "sg")[:, 0] if sp.shared.gated else None
         return ops.moe_combine(rows, h, rowidx, None if on_input else w, h.dtype, extra, gate)
 
     def checkpoint_map(self, pre: str) -> Dict[str, torch.Tensor]:
@@ -932,7 +1036,7 @@ class RoutedExperts(nn.Module):
             m[f"{pre}e{e}.up"] = self.w_in[e, :, -ff:].t()
             m[f"{pre}e{e}.down"] = self.w_down[e].t()
         if self.shared_inp is not None:
-            for n in ("gate", "up", "sg"):
+            for n in self.shared_inp.parts:
                 m[f"{pre}shared.{n}"] = self.shared_inp.slot(n)
             m[pre + "shared.down"] = self.shared_down
         return m

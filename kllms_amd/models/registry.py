@@ -34,7 +34,11 @@ def model_class(arch: str):
         from .bavesun import BavesunForCausalLM
 
         return BavesunForCausalLM
+    if arch == "dimuvik":
+        from .dimuvik import DimuvikForCausalLM
+
+        return DimuvikForCausalLM
     raise ValueError(f"no model registered for architecture {arch!r}")
 
 
-ARCHITECTURES = ("llama", "mixtral", "zutalix", "medilix", "mitunex", "pironex", "bavesun")
+ARCHITECTURES = ("llama", "mixtral", "zutalix", "medilix", "mitunex", "pironex", "bavesun", "dimuvik")

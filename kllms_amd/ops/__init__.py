@@ -522,20 +522,20 @@ def head_rmsnorm_gate(o, weight, gate, eps, gate_act, out_dtype):
 _SCORE_KINDS = {"softmax": 0, "sigmoid": 1, "top_softmax": 2}
 
 
-def moe_route(z, correction, top, group_count, group_keep, score="softmax", renormalize=True):
+def moe_route(z, correction, top, group_count, group_keep, score="softmax", renormalize=True, scale=1.0):
     """Routing from fp32 logits z [T, N]: (idx [T, top] int32, w [T, top] fp32)."""
     if _gpu(z):
         idx = torch.empty((z.shape[0], top), dtype=torch.int32, device=z.device)
         w = torch.empty((z.shape[0], top), dtype=torch.float32, device=z.device)
         _seq().moe_route(idx, w, _none(z, torch.int32), z, _none(z),
                          correction if correction is not None else _none(z), int(top), int(group_count),
-                         int(group_keep), 0, _SCORE_KINDS[score], bool(renormalize))
+                         int(group_keep), 0, _SCORE_KINDS[score], bool(renormalize), float(scale))
         return idx, w
-    return torch_ref.moe_route(z, correction, top, group_count, group_keep, score, renormalize)
+    return torch_ref.moe_route(z, correction, top, group_count, group_keep, score, renormalize, scale)
 
 
 def moe_route_rows(h, router, correction, top, group_count, group_keep, experts, all_experts_form,
-                   score="softmax", renormalize=True):
+                   score="softmax", renormalize=True, scale=1.0):
     """Router GEMV in fp32 + routing in one kernel. Returns (idx, w, rowidx);
     rowidx [T, top] (only when all_experts_form) addresses rows of the
     all-experts output [experts * T, W]: choice * T + row, -1 = identity."""
@@ -547,10 +547,10 @@ def moe_route_rows(h, router, correction, top, group_count, group_keep, experts,
         _seq().moe_route(idx, w, rowidx if rowidx is not None else _none(h, torch.int32), h, router,
                          correction if correction is not None else _none(router),
                          int(top), int(group_count), int(group_keep), int(experts),
-                         _SCORE_KINDS[score], bool(renormalize))
+                         _SCORE_KINDS[score], bool(renormalize), float(scale))
         return idx, w, rowidx
     z = torch.nn.functional.linear(h.float(), router)
-    idx, w = torch_ref.moe_route(z, correction, top, group_count, group_keep, score, renormalize)
+    idx, w = torch_ref.moe_route(z, correction, top, group_count, group_keep, score, renormalize, scale)
     rowidx = None
     if all_experts_form:
         t_idx = torch.arange(T, dtype=torch.int32, device=h.device).unsqueeze(1)
@@ -561,12 +561,12 @@ def moe_route_rows(h, router, correction, top, group_count, group_keep, experts,
 def moe_combine(rows, h, rowidx, w, out_dtype, extra=None, extra_gate=None):
     """Fixed-order sum of each row's chosen expert rows, weighted by w (None =
     unweighted), plus sigmoid(extra_gate[t]) * extra[t] when given
-    (extra_gate: a [T] view, any stride)."""
+    (extra_gate: a [T] view, any stride; None: plus extra[t])."""
     if _gpu(h):
         out = torch.empty(h.shape, dtype=out_dtype, device=h.device)
         _seq().moe_combine(out, rows, h, rowidx, w if w is not None else _none(h, torch.float32),
                            extra if extra is not None else _none(h),
-                           extra_gate if extra is not None else _none(h))
+                           extra_gate if extra_gate is not None else _none(h))
         return out
     return torch_ref.moe_combine(rows, h, rowidx, w, out_dtype, extra, extra_gate)
 
@@ -861,3 +861,111 @@ def add_cast(x, a, b, out_dtype):
         _seq().add_cast(_none(x, out_dtype) if out is x else out, x, a, b if b is not None else _none(a))
         return out
     return torch_ref.add_cast(x, a, b, out_dtype)
+
+
+def dyt_residual(x, a, post, nxt, out_dtype):
+    """x (fp32 stream, in place) += tanh(alpha a) w + b with post = (alpha, w,
+    b); returns tanh(alpha x) w + b with nxt, the next reader's input. a None:
+    x stays as it is."""
+    if _gpu(x):
+        out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
+        f = _none(x, torch.float32)
+        p = post if a is not None else (f, f, f)
+        _seq().dyt_residual(out, x, a if a is not None else _none(x, out_dtype), *p, *nxt)
+        return out
+    return torch_ref.dyt_residual(x, a, post, nxt, out_dtype)
+
+
+def rmsnorm_rows(x, weight, eps):
+    """RMS norm of a [T, C] row view, packed result in x's dtype."""
+    if _gpu(x):
+        out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+        _seq().rmsnorm_rows(out, x, weight, eps)
+        return out
+    return torch_ref.rmsnorm_rows(x, weight, eps)
+
+
+def conv_qkv_store(y, w, conv_state, state_slots, cu_seqlens, seg_start, token_seg, positions, q_cols, temp_coef,
+                   temp_every, k_cols=None, v_cols=None, k_cache=None, v_cache=None, slot_mapping=None, single=False):
+    """Short causal convolution of a fused projection's rows; k and v columns
+    into the paged caches, the q columns times the query temperature returned
+    packed [T, width]. ``single``: every segment is one row (the history is
+    updated by the same launch)."""
+    if _gpu(y):
+        q = torch.empty((y.shape[0], q_cols[1]), dtype=y.dtype, device=y.device)
+        has = k_cols is not None
+        e = _none(y)
+        ko, vo = (k_cols[0], v_cols[0]) if has else (0, 0)
+        _seq().conv_qkv_store(q, y, w, conv_state, state_slots, cu_seqlens, seg_start, token_seg, positions,
+                              int(q_cols[0]), float(temp_coef), int(temp_every), int(ko), int(vo),
+                              k_cache if has else e, v_cache if has else e,
+                              slot_mapping if has else _none(y, torch.long), bool(single))
+        return q
+    return torch_ref.conv_qkv_store(y, w, conv_state, state_slots, cu_seqlens, seg_start, positions, q_cols, temp_coef,
+                                    temp_every, k_cols, v_cols, k_cache, v_cache, slot_mapping)
+
+
+def diff_tile_rows(heads: int, kv_heads: int) -> int:
+    """Query rows per workgroup of the matrix-unit kernel: four tiles of 32
+    columns, of one head each, shared between consecutive rows and up to four
+    heads of a key/value head."""
+    r = heads // kv_heads
+    return 32 if r >= 3 else 128 // r
+
+
+def diff_tiles(segs, rows: int, device):
+    """Host metadata of attn_diff_paged for a step of segments
+    [(start position, rows)] in row order: (tiles [NT, 2] int32: first row,
+    row count — pieces of at most ``rows`` rows of a segment with two rows or
+    more, longest key ranges first; single [NS] int32: the rows of one-row
+    segments). Either may be empty."""
+    tiles, single, row0 = [], [], 0
+    for start, n in segs:
+        if n == 1:
+            single.append(row0)
+        else:
+            tiles += [(start + min(n, i + rows), row0 + i, min(rows, n - i)) for i in range(0, n, rows)]
+        row0 += n
+    tiles = [(r, n) for _, r, n in sorted(tiles, reverse=True)]
+    i32 = lambda x: torch.tensor(x, dtype=torch.int32, device=device)
+    return i32(tiles).reshape(-1, 2), i32(single)
+
+
+def diff_key_splits(rows: int, groups: int, reach: int) -> int:
+    """Workgroups that share one row's keys in the decode form: as many as
+    fill the chip, at most one per 64-key tile."""
+    tiles = max(1, (reach + 63) // 64)
+    return max(1, min(tiles, (512 + rows * groups - 1) // max(1, rows * groups), 64))
+
+
+def attn_diff_paged(q, k_cache, v_cache, block_tables, token_seg, positions, scale, lam, out_scale, eps, plan=None,
+                    use_mfma: bool = True, key_splits: int = 0):
+    """Differential attention over the paged cache (plain causal):
+    rms(softmax_1 v - lam softmax_2 v) * out_scale per head, [T, H, V].
+    GPU: bf16 goes through the matrix-unit kernels when the sizes fit them —
+    ``plan`` = diff_tiles() of the step, None = every row on its own (decode) —
+    and fp32 and other sizes through the plain kernel. ``key_splits``: see
+    diff_key_splits (0 = by that rule)."""
+    if _gpu(q):
+        T, H, V = q.shape[0], q.shape[1], v_cache.shape[3]
+        out = torch.empty((T, H, V), dtype=q.dtype, device=q.device)
+        f, i = _none(q, torch.float32), _none(q, torch.int32)
+        mfma = use_mfma and q.dtype == torch.bfloat16 and _seq().attn_diff_mfma_fits(q.shape[2] // 2, V)
+        args = (out, q, k_cache, v_cache, block_tables, token_seg, positions, float(scale), float(lam),
+                float(out_scale), float(eps))
+        if not mfma:
+            _seq().attn_diff_paged(*args, 0, i, f, f)
+            return out
+        tiles, single = plan if plan is not None else (i, i)
+        if tiles.numel():
+            _seq().attn_diff_paged(*args, 1, tiles, f, f)
+        n = T if plan is None else single.numel()
+        if n:
+            reach = block_tables.shape[1] * k_cache.shape[2]
+            ns = key_splits or diff_key_splits(n, k_cache.shape[1], reach)
+            part_o = torch.empty((n, H, 2, ns, V), dtype=torch.float32, device=q.device)
+            part_ml = torch.empty((n, H, 2, ns, 2), dtype=torch.float32, device=q.device)
+            _seq().attn_diff_paged(*args, 2, single, part_o, part_ml)
+        return out
+    return torch_ref.attn_diff_paged(q, k_cache, v_cache, block_tables, token_seg, positions, scale, lam, out_scale,
+                                     eps)

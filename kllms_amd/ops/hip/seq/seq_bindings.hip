@@ -70,7 +70,7 @@ void seq_launch_head_rmsnorm_gate(void*, const float*, const float*, const void*
 void seq_launch_token_shift_mix(void*, float*, const void*, const float*, void*, const int*, const int*,
                                 const int*, const int*, int, int, int, int, int, int, hipStream_t);
 void seq_launch_moe_route(int*, float*, int*, const float*, const void*, const float*, const float*, int, int, int,
-                          int, int, int, int, int, int, int, hipStream_t);
+                          int, int, int, int, int, int, float, int, hipStream_t);
 void seq_launch_moe_combine(void*, const void*, const void*, const int*, const float*, const void*, const void*,
                             int, int, int, int, int, hipStream_t);
 void seq_launch_wkv_recurrence(float*, const void*, const void*, const void*, const float*, const float*,
@@ -90,6 +90,16 @@ void seq_launch_gated_delta_rule(float*, const void*, const void*, const void*, 
                                  const float*, const float*, float*, float*, float*, float*, float*, float*,
                                  const int*, const int*, const int*, int, int, int, int, int, int, int, int, int,
                                  int, int, int, hipStream_t);
+void seq_launch_dyt_residual(void*, float*, const void*, const float*, const float*, const float*, const float*,
+                             const float*, const float*, int, int, int, hipStream_t);
+void seq_launch_rmsnorm_rows(void*, const void*, const float*, int, int, int, float, int, hipStream_t);
+void seq_launch_conv_qkv_store(void*, const void*, const float*, void*, const int*, const int*, const int*,
+                               const int*, const int64_t*, void*, void*, const int64_t*, int, int, int, int, int, int,
+                               int, int, int, int, int, int, int, int, int, float, int, int, int, hipStream_t);
+int seq_diff_mfma_fits(int, int);
+int seq_launch_attn_diff_paged(void*, const void*, const void*, const void*, const int*, const int*, const int64_t*,
+                               int, const int*, int, float, float, float, float, int, int, int, int, int, int, int, int,
+                               int, int, float*, float*, int, hipStream_t);
 }
 
 // dense varlen causal MFMA prefill kernel (ops/hip/attn_prefill.hip, also part
@@ -754,7 +764,7 @@ void token_shift_mix(torch::Tensor act, torch::Tensor f32, torch::Tensor h, torc
 // computed in the kernel. rowidx: empty, or [T, top] for the all-experts form over `experts` real experts.
 void moe_route(torch::Tensor idx, torch::Tensor w, torch::Tensor rowidx, torch::Tensor x, torch::Tensor router,
                torch::Tensor corr, int64_t top, int64_t gc, int64_t gk, int64_t experts, int64_t score_kind,
-               bool renorm) {
+               bool renorm, double wscale) {
   CHECK_I32C(idx); CHECK_F32C(w);
   TORCH_CHECK(x.dim() == 2 && x.is_cuda() && x.is_contiguous());
   const bool fused = router.numel() > 0;
@@ -782,10 +792,10 @@ void moe_route(torch::Tensor idx, torch::Tensor w, torch::Tensor rowidx, torch::
                        fused ? nullptr : x.data_ptr<float>(), fused ? x.data_ptr() : nullptr,
                        fused ? router.data_ptr<float>() : nullptr, has_corr ? corr.data_ptr<float>() : nullptr, T,
                        N, W, (int)top, (int)gc, (int)gk, (int)experts, (int)score_kind, renorm ? 1 : 0,
-                       fused ? f32flag(x) : 1, cur_stream());
+                       (float)wscale, fused ? f32flag(x) : 1, cur_stream());
 }
 
-// w: empty = unweighted; extra [T, W] / extra_gate ([T] view, any stride): empty = none
+// w: empty = unweighted; extra [T, W] / extra_gate ([T] view, any stride): empty = none (no gate: extra is added as it is)
 void moe_combine(torch::Tensor out, torch::Tensor rows, torch::Tensor h, torch::Tensor rowidx, torch::Tensor w,
                  torch::Tensor extra, torch::Tensor extra_gate) {
   CHECK_ACT(out); CHECK_ACT(rows); CHECK_ACT(h); CHECK_SAME(rows, out); CHECK_SAME(h, out);
@@ -797,14 +807,18 @@ void moe_combine(torch::Tensor out, torch::Tensor rows, torch::Tensor h, torch::
   if (weighted) { CHECK_F32C(w); TORCH_CHECK(w.numel() == rowidx.numel()); }
   const bool ex = extra.numel() > 0;
   if (ex) {
-    CHECK_ACT(extra); CHECK_SAME(extra, out); CHECK_ACT(extra_gate); CHECK_SAME(extra_gate, out);
+    CHECK_ACT(extra); CHECK_SAME(extra, out);
     TORCH_CHECK(extra.is_contiguous() && extra.dim() == 2 && extra.size(0) == T && extra.size(1) == W);
-    TORCH_CHECK(extra_gate.dim() == 1 && extra_gate.size(0) == T);
+  }
+  const bool gated = extra_gate.numel() > 0;
+  if (gated) {
+    CHECK_ACT(extra_gate); CHECK_SAME(extra_gate, out);
+    TORCH_CHECK(ex && extra_gate.dim() == 1 && extra_gate.size(0) == T);
   }
   if (T == 0) return;
   seq_launch_moe_combine(out.data_ptr(), rows.data_ptr(), h.data_ptr(), rowidx.data_ptr<int>(),
                          weighted ? w.data_ptr<float>() : nullptr, ex ? extra.data_ptr() : nullptr,
-                         ex ? extra_gate.data_ptr() : nullptr, ex ? (int)extra_gate.stride(0) : 0, T, W, top,
+                         gated ? extra_gate.data_ptr() : nullptr, gated ? (int)extra_gate.stride(0) : 0, T, W, top,
                          f32flag(out), cur_stream());
 }
 
@@ -1012,6 +1026,138 @@ void ssd_recurrence(torch::Tensor o, torch::Tensor x, torch::Tensor Bm, torch::T
                             cur_stream());
 }
 
+// ---- dynamic-tanh norms, differential attention ----------------------------------
+
+// a / alpha_p / w_p / b_p empty: the stream stays as it is
+void dyt_residual(torch::Tensor out, torch::Tensor x, torch::Tensor a, torch::Tensor alpha_p, torch::Tensor w_p,
+                  torch::Tensor b_p, torch::Tensor alpha_n, torch::Tensor w_n, torch::Tensor b_n) {
+  CHECK_ACT(out); CHECK_F32C(x); CHECK_F32C(alpha_n); CHECK_F32C(w_n); CHECK_F32C(b_n);
+  TORCH_CHECK(x.dim() == 2 && out.is_contiguous() && out.sizes() == x.sizes());
+  const int T = x.size(0), W = x.size(1);
+  TORCH_CHECK(alpha_n.numel() == 1 && w_n.numel() == W && b_n.numel() == W);
+  const bool has = a.numel() > 0;
+  if (has) {
+    CHECK_ACT(a); CHECK_SAME(a, out); CHECK_F32C(alpha_p); CHECK_F32C(w_p); CHECK_F32C(b_p);
+    TORCH_CHECK(a.is_contiguous() && a.sizes() == x.sizes());
+    TORCH_CHECK(alpha_p.numel() == 1 && w_p.numel() == W && b_p.numel() == W);
+  }
+  if (x.numel() == 0) return;
+  seq_launch_dyt_residual(out.data_ptr(), x.data_ptr<float>(), has ? a.data_ptr() : nullptr,
+                          has ? alpha_p.data_ptr<float>() : nullptr, has ? w_p.data_ptr<float>() : nullptr,
+                          has ? b_p.data_ptr<float>() : nullptr, alpha_n.data_ptr<float>(), w_n.data_ptr<float>(),
+                          b_n.data_ptr<float>(), T, W, f32flag(out), cur_stream());
+}
+
+void rmsnorm_rows(torch::Tensor out, torch::Tensor x, torch::Tensor w, double eps) {
+  CHECK_ACT(out); CHECK_ACT(x); CHECK_SAME(x, out); CHECK_ROWS2(x); CHECK_F32C(w);
+  TORCH_CHECK(out.is_contiguous() && out.sizes() == x.sizes() && w.numel() == x.size(1));
+  if (x.numel() == 0) return;
+  seq_launch_rmsnorm_rows(out.data_ptr(), x.data_ptr(), w.data_ptr<float>(), (int)x.size(0), (int)x.size(1),
+                          (int)x.stride(0), (float)eps, f32flag(out), cur_stream());
+}
+
+// y [T, C] rows of a fused projection; q_out [T, width] = columns qo..; caches [NB, G, BS, D | V] take the
+// columns from ko and vo (caches empty: q only). single: every segment is one row
+void conv_qkv_store(torch::Tensor q_out, torch::Tensor y, torch::Tensor w, torch::Tensor hist, torch::Tensor slots,
+                    torch::Tensor cu, torch::Tensor seg_start, torch::Tensor token_seg, torch::Tensor positions,
+                    int64_t qo, double coef, int64_t every, int64_t ko, int64_t vo, torch::Tensor k_cache,
+                    torch::Tensor v_cache, torch::Tensor slot_map, bool single) {
+  CHECK_ACT(y); CHECK_ROWS2(y); CHECK_SAME(q_out, y); CHECK_SAME(hist, y); CHECK_F32C(w); CHECK_I32C(token_seg);
+  CHECK_I64C(positions);
+  check_segments(slots, cu, seg_start, hist);
+  const int T = y.size(0), C = y.size(1), B = slots.numel();
+  TORCH_CHECK(w.dim() == 2 && w.size(1) == C && w.size(0) >= 1 && w.size(0) <= 16, "1..16 convolution taps supported");
+  const int K = w.size(0);
+  TORCH_CHECK(hist.dim() == 3 && hist.size(1) == K - 1 && hist.size(2) == C);
+  TORCH_CHECK(q_out.is_cuda() && q_out.is_contiguous() && q_out.dim() == 2 && q_out.size(0) == T);
+  const int64_t qn = q_out.size(1);
+  TORCH_CHECK(qo >= 0 && qo + qn <= C && every >= 1 && every < (1LL << 31));
+  TORCH_CHECK(token_seg.numel() == T && positions.numel() == T && (!single || B == T));
+  int64_t kn = 0, vn = 0;
+  int G = 1, D2 = 1, V = 1, BS = 1;
+  const bool has = k_cache.numel() > 0;
+  if (has) {
+    CHECK_SAME(k_cache, y); CHECK_SAME(v_cache, y); CHECK_I64C(slot_map);
+    TORCH_CHECK(k_cache.is_cuda() && v_cache.is_cuda() && k_cache.is_contiguous() && v_cache.is_contiguous() &&
+                k_cache.dim() == 4 && v_cache.dim() == 4);
+    G = k_cache.size(1); BS = k_cache.size(2); D2 = k_cache.size(3); V = v_cache.size(3);
+    kn = (int64_t)G * D2; vn = (int64_t)G * V;
+    TORCH_CHECK(v_cache.size(0) == k_cache.size(0) && v_cache.size(1) == G && v_cache.size(2) == BS);
+    TORCH_CHECK(ko >= 0 && ko + kn <= C && vo >= 0 && vo + vn <= C && slot_map.numel() == T);
+    TORCH_CHECK((ko >= qo + qn || ko + kn <= qo) && (vo >= qo + qn || vo + vn <= qo) && (vo >= ko + kn || vo + vn <= ko),
+                "column ranges overlap");
+  }
+  if (T == 0 || B == 0) return;
+  seq_launch_conv_qkv_store(q_out.data_ptr(), y.data_ptr(), w.data_ptr<float>(), hist.data_ptr(), slots.data_ptr<int>(),
+                            cu.data_ptr<int>(), seg_start.data_ptr<int>(), token_seg.data_ptr<int>(),
+                            positions.data_ptr<int64_t>(), has ? k_cache.data_ptr() : nullptr,
+                            has ? v_cache.data_ptr() : nullptr, has ? slot_map.data_ptr<int64_t>() : nullptr, T, B, C, K,
+                            (int)y.stride(0), (int)qo, (int)qn, (int)ko, (int)kn, (int)vo, (int)vn, D2, V, G, BS,
+                            (float)coef, (int)every, single ? 1 : 0, f32flag(y), cur_stream());
+}
+
+bool attn_diff_mfma_fits(int64_t D, int64_t V) { return seq_diff_mfma_fits((int)D, (int)V) != 0; }
+
+// heads of one key/value head that a query-tile workgroup serves side by side; its rows are 32 * (4 / that)
+static int diff_tile_heads(int R) { return R >= 3 ? 4 : R; }
+
+// q [T, H, 2 D] row view, out [T, H, V]. form 0: the plain kernel. form 1: rows = query tiles [n, 2] int32 (first
+// row, row count), each within one segment. form 2: rows = list of single rows or empty (= all T), partial results
+// part_o [n, H, 2, ns, V], part_ml [n, H, 2, ns, 2] fp32. Forms 1 and 2: bf16 (the host built the row lists; they
+// are not re-read here)
+void attn_diff_paged(torch::Tensor out, torch::Tensor q, torch::Tensor k_cache, torch::Tensor v_cache,
+                     torch::Tensor block_tables, torch::Tensor token_seg, torch::Tensor positions, double scale,
+                     double lam, double oscale, double eps, int64_t form, torch::Tensor rows, torch::Tensor part_o,
+                     torch::Tensor part_ml) {
+  CHECK_ACT(q); CHECK_ROWS3(q); CHECK_SAME(out, q); CHECK_SAME(k_cache, q); CHECK_SAME(v_cache, q);
+  CHECK_I32C(token_seg); CHECK_I64C(positions);
+  TORCH_CHECK(block_tables.is_cuda() && block_tables.scalar_type() == at::kInt && block_tables.dim() == 2 &&
+              block_tables.stride(1) == 1);
+  TORCH_CHECK(out.is_cuda() && out.is_contiguous() && k_cache.is_cuda() && v_cache.is_cuda() && k_cache.is_contiguous() &&
+              v_cache.is_contiguous() && k_cache.dim() == 4 && v_cache.dim() == 4);
+  const int T = q.size(0), H = q.size(1), D = (int)(q.size(2) / 2);
+  const int G = k_cache.size(1), BS = k_cache.size(2), V = v_cache.size(3);
+  TORCH_CHECK(q.size(2) == 2 * D && k_cache.size(3) == 2 * D && H % G == 0 && v_cache.size(0) == k_cache.size(0) &&
+              v_cache.size(1) == G && v_cache.size(2) == BS);
+  TORCH_CHECK(out.numel() == (int64_t)T * H * V && token_seg.numel() == T && positions.numel() == T);
+  TORCH_CHECK(D >= 1 && D <= 4096 && V >= 1 && V <= 512, "head sizes of the differential attention kernels");
+  TORCH_CHECK(k_cache.size(0) * G * BS < (1LL << 31));
+  if (T == 0) return;
+  const int R = H / G;
+  int n = T, hb = 1, ns = 1;
+  const bool listed = rows.numel() > 0;
+  if (listed) CHECK_I32C(rows);
+  if (form != 0) {
+    TORCH_CHECK(q.scalar_type() == at::kBFloat16 && seq_diff_mfma_fits(D, V), "sizes of the matrix-unit kernels");
+    TORCH_CHECK(q.stride(0) % 8 == 0 && (reinterpret_cast<uintptr_t>(q.data_ptr()) & 15) == 0 &&
+                (reinterpret_cast<uintptr_t>(k_cache.data_ptr()) & 15) == 0 &&
+                (reinterpret_cast<uintptr_t>(v_cache.data_ptr()) & 15) == 0, "16-byte aligned rows");
+  }
+  if (form == 1) {
+    TORCH_CHECK(listed && rows.dim() == 2 && rows.size(1) == 2 && rows.size(0) <= T);
+    n = rows.size(0);
+    hb = diff_tile_heads(R);
+  } else if (form == 2) {
+    if (listed) { TORCH_CHECK(rows.dim() == 1 && rows.numel() <= T); n = rows.numel(); }
+    hb = R < 32 ? R : 32;
+    CHECK_F32C(part_o); CHECK_F32C(part_ml);
+    TORCH_CHECK(part_o.dim() == 5 && part_o.size(0) == n && part_o.size(1) == H && part_o.size(2) == 2 &&
+                part_o.size(4) == V);
+    ns = part_o.size(3);
+    TORCH_CHECK(ns >= 1 && ns <= 64 && part_ml.numel() == (int64_t)n * H * 2 * ns * 2);
+  } else {
+    TORCH_CHECK(form == 0 && !listed);
+  }
+  TORCH_CHECK(n <= 65535 || form == 0, "too many row tiles for one launch");
+  const int err = seq_launch_attn_diff_paged(
+      out.data_ptr(), q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(), block_tables.data_ptr<int>(),
+      token_seg.data_ptr<int>(), positions.data_ptr<int64_t>(), (int)form, listed ? rows.data_ptr<int>() : nullptr, n,
+      (float)scale, (float)lam, (float)oscale, (float)eps, T, H, G, D, V, BS, (int)block_tables.stride(0),
+      (int)q.stride(0), hb, ns, form == 2 ? part_o.data_ptr<float>() : nullptr,
+      form == 2 ? part_ml.data_ptr<float>() : nullptr, f32flag(q), cur_stream());
+  TORCH_CHECK(err == 0, "attn_diff_paged launch: ", hipGetErrorString((hipError_t)err));
+}
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("embed_rmsnorm", &embed_rmsnorm);
   m.def("rmsnorm_cast", &rmsnorm_cast);
@@ -1053,4 +1199,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("qk_fullnorm_rope_store", &qk_fullnorm_rope_store);
   m.def("pool_kv_update", &pool_kv_update);
   m.def("ssd_recurrence", &ssd_recurrence);
+  m.def("dyt_residual", &dyt_residual);
+  m.def("rmsnorm_rows", &rmsnorm_rows);
+  m.def("conv_qkv_store", &conv_qkv_store);
+  m.def("attn_diff_mfma_fits", &attn_diff_mfma_fits);
+  m.def("attn_diff_paged", &attn_diff_paged);
 }

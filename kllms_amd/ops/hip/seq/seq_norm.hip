@@ -388,6 +388,72 @@ __global__ void scale_softcap_kernel(float* __restrict__ z, int64_t n, float sca
   }
 }
 
+// ---- dynamic-tanh norm: tanh(alpha v) w + b, no statistics -------------------------
+// x (fp32 stream) += tanh(alpha_p a) w_p + b_p (a == nullptr: x as it is), then
+// out = tanh(alpha_n x) w_n + b_n. A thread keeps VEC columns of both norms in
+// registers and walks the rows blockIdx.y, + gridDim.y, ...
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256) dyt_residual_kernel(
+    T* __restrict__ out, float* __restrict__ x, const T* __restrict__ a, const float* __restrict__ alpha_p,
+    const float* __restrict__ w_p, const float* __restrict__ b_p, const float* __restrict__ alpha_n,
+    const float* __restrict__ w_n, const float* __restrict__ b_n, int T_, int W) {
+  const int c = (blockIdx.x * blockDim.x + threadIdx.x) * VEC;
+  if (c >= W) return;
+  float wp[VEC], bp[VEC], wn[VEC], bn[VEC];
+  const float an = alpha_n[0], ap = a != nullptr ? alpha_p[0] : 0.f;
+  if constexpr (VEC == 8) {
+    ld8(w_n + c, wn); ld8(b_n + c, bn);
+    if (a != nullptr) { ld8(w_p + c, wp); ld8(b_p + c, bp); }
+  } else {
+    wn[0] = w_n[c]; bn[0] = b_n[c];
+    if (a != nullptr) { wp[0] = w_p[c]; bp[0] = b_p[c]; }
+  }
+  for (int64_t t = blockIdx.y; t < T_; t += gridDim.y) {
+    float xv[VEC], av[VEC];
+    if constexpr (VEC == 8) {
+      ld8(x + t * W + c, xv);
+      if (a != nullptr) ld8(a + t * W + c, av);
+    } else {
+      xv[0] = x[t * W + c];
+      if (a != nullptr) av[0] = ldf(a + t * W + c);
+    }
+    if (a != nullptr) {
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) xv[e] += tanhf(ap * av[e]) * wp[e] + bp[e];
+      if constexpr (VEC == 8) st8(x + t * W + c, xv); else x[t * W + c] = xv[0];
+    }
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) xv[e] = tanhf(an * xv[e]) * wn[e] + bn[e];
+    if constexpr (VEC == 8) st8(out + t * W + c, xv); else stf(out + t * W + c, xv[0]);
+  }
+}
+
+// RMS norm of rows in the activation type (free row stride), one wave per row
+template <typename T, int VEC>
+__global__ void __launch_bounds__(256) rmsnorm_rows_kernel(T* __restrict__ out, const T* __restrict__ x,
+                                                           const float* __restrict__ w, int T_, int C, int x_stride,
+                                                           float eps) {
+  const int lane = threadIdx.x & (WAVE - 1);
+  const int64_t t = (int64_t)blockIdx.x * (256 / WAVE) + threadIdx.x / WAVE;
+  if (t >= T_) return;
+  const T* row = x + t * x_stride;
+  float ss = 0.f;
+  for (int c = lane * VEC; c < C; c += WAVE * VEC) {
+    float v[VEC];
+    if constexpr (VEC == 8) ld8(row + c, v); else v[0] = ldf(row + c);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) ss += v[e] * v[e];
+  }
+  const float r = 1.0f / sqrtf(wave_sum(ss) / (float)C + eps);
+  for (int c = lane * VEC; c < C; c += WAVE * VEC) {
+    float v[VEC], wv[VEC];
+    if constexpr (VEC == 8) { ld8(row + c, v); ld8(w + c, wv); } else { v[0] = ldf(row + c); wv[0] = w[c]; }
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v[e] *= r * wv[e];
+    if constexpr (VEC == 8) st8(out + t * C + c, v); else stf(out + t * C + c, v[0]);
+  }
+}
+
 #define DISPATCH_T(is_f32, ...)                                  \
   if (is_f32) { typedef float T; __VA_ARGS__ } else { typedef bfraw T; __VA_ARGS__ }
 
@@ -511,4 +577,33 @@ extern "C" void seq_launch_gated_act(void* out, const void* gate, const void* up
   const int grid = (int)((n + 255) / 256 < 4096 ? (n + 255) / 256 : 4096);
   DISPATCH_T(is_f32, hipLaunchKernelGGL(clamped_glu_kernel<T>, dim3(grid), dim3(256), 0, st, (T*)out,
                                         (const T*)gate, (const T*)up, n, cols, stride, limit, alpha, up_bias);)
+}
+
+extern "C" void seq_launch_dyt_residual(void* out, float* x, const void* a, const float* alpha_p, const float* w_p,
+                                        const float* b_p, const float* alpha_n, const float* w_n, const float* b_n,
+                                        int T_, int W, int is_f32, hipStream_t st) {
+  const bool v8 = W % 8 == 0 && aligned16(out) && aligned16(x) && aligned16(w_n) && aligned16(b_n) &&
+                  (a == nullptr || (aligned16(a) && aligned16(w_p) && aligned16(b_p)));
+  const int cols = v8 ? W / 8 : W;
+  const int threads = cols >= 256 ? 256 : (cols + WAVE - 1) / WAVE * WAVE;
+  const int gx = (cols + threads - 1) / threads;
+  int gy = (8192 * 256 / threads + gx - 1) / gx;
+  if (gy > T_) gy = T_;
+  if (gy > 65535) gy = 65535;
+  DISPATCH_T(is_f32,
+             if (v8) hipLaunchKernelGGL((dyt_residual_kernel<T, 8>), dim3(gx, gy), dim3(threads), 0, st, (T*)out, x,
+                                        (const T*)a, alpha_p, w_p, b_p, alpha_n, w_n, b_n, T_, W);
+             else hipLaunchKernelGGL((dyt_residual_kernel<T, 1>), dim3(gx, gy), dim3(threads), 0, st, (T*)out, x,
+                                     (const T*)a, alpha_p, w_p, b_p, alpha_n, w_n, b_n, T_, W);)
+}
+
+extern "C" void seq_launch_rmsnorm_rows(void* out, const void* x, const float* w, int T_, int C, int x_stride,
+                                        float eps, int is_f32, hipStream_t st) {
+  const bool v8 = C % 8 == 0 && x_stride % 8 == 0 && aligned16(out) && aligned16(x) && aligned16(w);
+  const int rows = 256 / WAVE;
+  DISPATCH_T(is_f32,
+             if (v8) hipLaunchKernelGGL((rmsnorm_rows_kernel<T, 8>), dim3((T_ + rows - 1) / rows), dim3(256), 0, st,
+                                        (T*)out, (const T*)x, w, T_, C, x_stride, eps);
+             else hipLaunchKernelGGL((rmsnorm_rows_kernel<T, 1>), dim3((T_ + rows - 1) / rows), dim3(256), 0, st,
+                                     (T*)out, (const T*)x, w, T_, C, x_stride, eps);)
 }

@@ -288,7 +288,8 @@ __global__ void shift_state_update_kernel(const T* __restrict__ h, T* __restrict
 // logits and renormalised weights are the softmax over the chosen ones); the
 // outputs form `gc` equal groups of neighbours, a group's score is its largest
 // c, the best `gk` groups stay eligible; the `top` eligible outputs with the
-// largest c are chosen (ties: the lower index). w = chosen s / (sum + 1e-20).
+// largest c are chosen (ties: the lower index). w = wscale * chosen s, with
+// renorm divided by (their sum + 1e-20).
 // The logits come from z [T, N], or (z == nullptr) are computed here in fp32
 // as router [N, W] times the row of h. rowidx (optional) receives, for the
 // all-experts form with E real experts over T_ rows, choice * T_ + row for a
@@ -301,7 +302,7 @@ __global__ void __launch_bounds__(256) moe_route_kernel(int* __restrict__ idx, f
                                                         const float* __restrict__ router,
                                                         const float* __restrict__ corr, int N, int W, int top,
                                                         int gc, int gk, int E, int T_, int vec,
-                                                        int score_kind, int renorm) {
+                                                        int score_kind, int renorm, float wscale) {
   __shared__ float cs[ROUTE_MAX_N], ss[ROUTE_MAX_N], gmax[ROUTE_MAX_N], zs[ROUTE_MAX_N];
   __shared__ int ok[ROUTE_MAX_N];
   const int64_t t = blockIdx.x;
@@ -398,18 +399,18 @@ __global__ void __launch_bounds__(256) moe_route_kernel(int* __restrict__ idx, f
     }
     __syncthreads();
   }
-  if (wave == 0 && lane < top) wout[t * top + lane] = renorm ? mine / (wsum + 1e-20f) : mine;
+  if (wave == 0 && lane < top) wout[t * top + lane] = (renorm ? mine / (wsum + 1e-20f) : mine) * wscale;
 }
 
 // ---- combine: out[t] = sum_j w[t,j] * (rowidx[t,j] >= 0 ? rows[rowidx[t,j]] : h[t]) ------
-// w == nullptr: unweighted. extra != nullptr: + sigmoid(extra_gate[t]) * extra[t].
+// w == nullptr: unweighted. extra != nullptr: + sigmoid(extra_gate[t]) * extra[t] (extra_gate == nullptr: + extra[t]).
 template <typename T>
 __global__ void moe_combine_kernel(T* __restrict__ out, const T* __restrict__ rows, const T* __restrict__ h,
                                    const int* __restrict__ rowidx, const float* __restrict__ w,
                                    const T* __restrict__ extra, const T* __restrict__ extra_gate,
                                    int gate_stride, int W, int top) {
   const int64_t t = blockIdx.x;
-  const float eg = extra != nullptr ? sigmoid_exact(ldf(extra_gate + t * gate_stride)) : 0.f;
+  const float eg = extra_gate != nullptr ? sigmoid_exact(ldf(extra_gate + t * gate_stride)) : 1.f;
   for (int i = threadIdx.x; i < W; i += blockDim.x) {
     float acc = 0.f;
     for (int j = 0; j < top; ++j) {
@@ -429,7 +430,7 @@ __global__ void moe_combine_v8_kernel(T* __restrict__ out, const T* __restrict__
                                       const T* __restrict__ extra, const T* __restrict__ extra_gate,
                                       int gate_stride, int W, int top) {
   const int64_t t = blockIdx.x;
-  const float eg = extra != nullptr ? sigmoid_exact(ldf(extra_gate + t * gate_stride)) : 0.f;
+  const float eg = extra_gate != nullptr ? sigmoid_exact(ldf(extra_gate + t * gate_stride)) : 1.f;
   for (int i = threadIdx.x * 8; i < W; i += blockDim.x * 8) {
     float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, v[8];
     for (int j = 0; j < top; ++j) {
@@ -575,13 +576,13 @@ extern "C" void seq_launch_token_shift_mix(void* act, float* f32, const void* h,
 
 extern "C" void seq_launch_moe_route(int* idx, float* w, int* rowidx, const float* z, const void* h,
                                      const float* router, const float* corr, int T_, int N, int W, int top,
-                                     int gc, int gk, int E, int score_kind, int renorm, int is_f32,
-                                     hipStream_t st) {
+                                     int gc, int gk, int E, int score_kind, int renorm, float wscale,
+                                     int is_f32, hipStream_t st) {
   const int vec = (h != nullptr && W % 8 == 0 && aligned16(h) && aligned16(router)) ? 1 : 0;
   const int threads = h != nullptr ? 256 : WAVE;
   DISPATCH_T(is_f32, hipLaunchKernelGGL(moe_route_kernel<T>, dim3(T_), dim3(threads), 0, st, idx, w, rowidx, z,
                                         (const T*)h, router, corr, N, W, top, gc, gk, E, T_, vec, score_kind,
-                                        renorm);)
+                                        renorm, wscale);)
 }
 
 extern "C" void seq_launch_moe_combine(void* out, const void* rows, const void* h, const int* rowidx,

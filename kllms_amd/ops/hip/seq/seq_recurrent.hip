@@ -638,3 +638,12 @@ extern "C" void seq_launch_gated_delta_rule(float* o, const void* q, const void*
                                                    st, o, qn, kn, gd, vf, bt, state, slots, cu, seg_start, H, G,
                                                    D, V);))
 }
+
+// the carried history alone, for kernels of other files that convolve by themselves
+extern "C" void seq_launch_conv_state_update(const void* x, void* conv_state, const int* slots, const int* cu,
+                                             const int* seg_start, int B, int C, int K, int x_stride, int is_f32,
+                                             hipStream_t st) {
+  const int grid = (int)(((int64_t)B * C + 255) / 256);
+  DISPATCH_T(is_f32, hipLaunchKernelGGL(conv_state_update_kernel<T>, dim3(grid), dim3(256), 0, st, (const T*)x,
+                                        (T*)conv_state, slots, cu, seg_start, B, C, K, x_stride);)
+}

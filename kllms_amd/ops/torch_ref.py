@@ -669,13 +669,14 @@ def gated_act(gate, up, limit: float, alpha: float, up_bias: float) -> torch.Ten
     return (g * torch.sigmoid(alpha * g) * (u + up_bias)).to(gate.dtype)
 
 
-def moe_route(z, correction, top, group_count, group_keep, score="softmax", renormalize=True):
+def moe_route(z, correction, top, group_count, group_keep, score="softmax", renormalize=True, scale=1.0):
     """z [T, N] fp32 router logits. Scores s = softmax(z) over the outputs,
     sigmoid(z) of each, or ("top_softmax") exp(z - max z); the choice is made
     on c = s + correction (None = no correction; "top_softmax": on z + correction) among the experts of the ``group_keep`` groups (of
     ``group_count`` equal runs of neighbours) whose largest c is largest;
     ties go to the lower index. Returns (idx [T, top] int32, w [T, top] fp32
-    = chosen s, divided by (their sum + 1e-20) if ``renormalize``)."""
+    = chosen s, divided by (their sum + 1e-20) if ``renormalize``, times
+    ``scale``)."""
     T, N = z.shape
     zf = z.float()
     if score == "top_softmax":
@@ -695,13 +696,14 @@ def moe_route(z, correction, top, group_count, group_keep, score="softmax", reno
     w = s.gather(1, idx)
     if renormalize:
         w = w / (w.sum(-1, keepdim=True) + 1e-20)
-    return idx.to(torch.int32), w
+    return idx.to(torch.int32), w * scale
 
 
 def moe_combine(rows, h, rowidx, w, out_dtype, extra=None, extra_gate=None) -> torch.Tensor:
     """out[t] = sum_j w[t, j] * (rows[rowidx[t, j]] if rowidx >= 0 else h[t]),
     summed in the order j = 0, 1, ... in fp32 (w None = all ones); then
-    + sigmoid(extra_gate[t]) * extra[t] when given. rows [R, W], h [T, W]."""
+    + sigmoid(extra_gate[t]) * extra[t] when given (extra_gate None: + extra[t]).
+    rows [R, W], h [T, W]."""
     T, top = rowidx.shape
     out = torch.zeros(T, h.shape[1], dtype=torch.float32, device=h.device)
     hf = h.float()
@@ -710,7 +712,8 @@ def moe_combine(rows, h, rowidx, w, out_dtype, extra=None, extra_gate=None) -> t
         src = torch.where((ri >= 0)[:, None], rows[ri.clamp(min=0)].float(), hf)
         out += src if w is None else w[:, j:j + 1].float() * src
     if extra is not None:
-        out += torch.sigmoid(extra_gate.float()).reshape(T, 1) * extra.float()
+        g = 1.0 if extra_gate is None else torch.sigmoid(extra_gate.float()).reshape(T, 1)
+        out += g * extra.float()
     return out.to(out_dtype)
 
 
@@ -1054,3 +1057,79 @@ def gate_group_rmsnorm(o, weight, gate, eps, out_dtype) -> torch.Tensor:
     y = o.float() * torch.nn.functional.silu(gate.float()).view(T, Gn, S)
     y = y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps)
     return (y.reshape(T, Gn * S) * weight.float()).to(out_dtype)
+
+
+# --- dynamic-tanh norms; plain short convolutions of the projections; differential
+# attention ------------------------------------------------------------------------
+
+def _dyt(v, alpha, w, b) -> torch.Tensor:
+    return torch.tanh(alpha.float() * v) * w.float() + b.float()
+
+
+def dyt_residual(x, a, post, nxt, out_dtype) -> torch.Tensor:
+    """x (fp32, in place) += tanh(alpha a) w + b with post = (alpha, w, b), or
+    x as it is when a is None; returns tanh(alpha x) w + b with nxt, cast."""
+    if a is not None:
+        x.add_(_dyt(a.float(), *post))
+    return _dyt(x, *nxt).to(out_dtype)
+
+
+def rmsnorm_rows(x, weight, eps) -> torch.Tensor:
+    """RMS norm of a [T, C] row view in x's dtype (statistics and product in fp32)."""
+    return rmsnorm_cast(x, weight, eps, x.dtype)
+
+
+def conv_qkv_store(y, w, conv_state, state_slots, cu_seqlens, seg_start, positions, q_cols, temp_coef, temp_every,
+                   k_cols, v_cols, k_cache, v_cache, slot_mapping) -> torch.Tensor:
+    """Per-channel causal convolution over time of a projection's rows
+    y [T, C] (w [K, C] taps-major, last row = current token; conv_state
+    [slots, K-1, C] holds the last K-1 rows and is updated), without an
+    activation. (offset, width) column ranges: the k and v columns go to the
+    paged caches [NB, G, BS, D | Dv] at the flat slots, the q columns times
+    1 + temp_coef ln(floor((p + 1) / temp_every) + 1) are returned."""
+    T, C = y.shape
+    K = w.shape[0]
+    z = torch.empty(T, C, dtype=torch.float32, device=y.device)
+    cu, st, sl = cu_seqlens.tolist(), seg_start.tolist(), state_slots.tolist()
+    wf = w.float()
+    for b in range(len(sl)):
+        s, e = cu[b], cu[b + 1]
+        if e == s:
+            continue
+        hist = conv_state[sl[b]].float() if st[b] > 0 else torch.zeros(K - 1, C, device=y.device)
+        ext = torch.cat([hist, y[s:e].float()], 0)
+        z[s:e] = sum(ext[j:j + (e - s)] * wf[j] for j in range(K))
+        if K > 1:
+            conv_state[sl[b]] = ext[ext.shape[0] - (K - 1):].to(conv_state.dtype)
+    if k_cols is not None:
+        G, BS = k_cache.shape[1], k_cache.shape[2]
+        blk, off = slot_mapping // BS, slot_mapping % BS
+        for (o, n), cache in ((k_cols, k_cache), (v_cols, v_cache)):
+            cache[blk, :, off] = z[:, o:o + n].view(T, G, -1).to(cache.dtype)
+    temp = 1.0 + temp_coef * torch.log(((positions + 1) // temp_every + 1).float())
+    return (z[:, q_cols[0]:q_cols[0] + q_cols[1]] * temp[:, None]).to(y.dtype)
+
+
+def attn_diff_paged(q, k_cache, v_cache, block_tables, token_seg, positions, scale, lam, out_scale, eps) -> torch.Tensor:
+    """Differential attention over the paged cache, plain causal. q [T, H, 2 D]
+    (map 1 | map 2 of every head), k_cache [NB, G, BS, 2 D] likewise, v_cache
+    [NB, G, BS, V]. Per head a_m = softmax(q_m . k_m scale) v for both maps,
+    o = a_1 - lam a_2, out = o / sqrt(mean(o^2) + eps) * out_scale; fp32 up to
+    the cast to q's dtype. Returns [T, H, V]."""
+    T, H, D2 = q.shape
+    D = D2 // 2
+    G, BS, V = k_cache.shape[1], k_cache.shape[2], v_cache.shape[3]
+    out = torch.empty(T, H, V, dtype=q.dtype, device=q.device)
+    seg, pos = token_seg.tolist(), positions.tolist()
+    for t in range(T):
+        n = pos[t] + 1
+        j = torch.arange(n, device=q.device)
+        blk = block_tables[seg[t]].long()[j // BS]
+        k = k_cache[blk, :, j % BS].float().view(n, G, 2, D)
+        v = v_cache[blk, :, j % BS].float()                                   # [n, G, V]
+        qt = q[t].float().view(G, H // G, 2, D)
+        s = torch.einsum("ghmd,ngmd->ghmn", qt, k) * scale
+        a = torch.einsum("ghmn,ngv->ghmv", torch.softmax(s, -1), v)
+        o = (a[:, :, 0] - lam * a[:, :, 1]).reshape(H, V)
+        out[t] = (o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * out_scale).to(q.dtype)
+    return out
