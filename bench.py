@@ -212,7 +212,7 @@ def main():
                     help="prefill/decode tok/s of the hybrid families beside the dense Llama stack of equal shape")
     ap.add_argument("--families", type=str, default="llama,zutalix,medilix",
                     help="--compare-families: model families to time, in order "
-                         "(llama, zutalix, medilix, mitunex, pironex, bavesun)")
+                         "(llama, zutalix, medilix, mitunex, pironex, bavesun, dimuvik)")
     ap.add_argument("--sizes", type=str, default="1b-l6,8b-l6", help="--compare-families: preset size suffixes")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=3)
