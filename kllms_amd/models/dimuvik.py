@@ -7,8 +7,9 @@ layer), and latent attention with a query latent and a sink; the feed-forward
 is a squared-relu layer, routed silu experts with a shared expert, or absent.
 The LM head is a matrix of its own.
 
-Kernel plan of one layer: mixer on h -> dyt_residual (post-norm, residual add,
-the next reader's norm, cast) -> feed-forward -> dyt_residual.
+Kernel plan: embed_dyt (the stream and the first norm), then per layer: mixer
+on h -> dyt_residual (post-norm, residual add, the next reader's norm, cast)
+-> feed-forward -> dyt_residual.
 """
 
 from __future__ import annotations
@@ -112,11 +113,9 @@ class DimuvikForCausalLM(ListedLayerLM):
     def forward_hidden(self, input_ids: torch.Tensor, batch: ForwardBatch) -> torch.Tensor:
         assert batch.seg_start is not None, "this model takes segment batches"
         states: List[LayerState] = batch.kv_caches
-        x = ops.embed_bigram(input_ids, self.embed_tokens.weight, None, self.cfg.embed_scale, 0, 0, 0, None,
-                             batch.state_slots, batch.cu_seqlens, batch.seg_start, batch.token_seg)
         # the norm of whatever reads the stream after each layer
         nxt = [layer.norm1.args for layer in self.layers] + [self.final_norm.args]
-        h = ops.dyt_residual(x, None, None, nxt[0], self.dtype)
+        x, h = ops.embed_dyt(input_ids, self.embed_tokens.weight, self.cfg.embed_scale, nxt[0])
         for i, layer in enumerate(self.layers):
             a = layer.mix(h, batch, states[i])
             if layer.mlp is not None:

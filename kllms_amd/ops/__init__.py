@@ -865,15 +865,23 @@ def add_cast(x, a, b, out_dtype):
 
 def dyt_residual(x, a, post, nxt, out_dtype):
     """x (fp32 stream, in place) += tanh(alpha a) w + b with post = (alpha, w,
-    b); returns tanh(alpha x) w + b with nxt, the next reader's input. a None:
-    x stays as it is."""
+    b); returns tanh(alpha x) w + b with nxt, the next reader's input."""
     if _gpu(x):
         out = torch.empty(x.shape, dtype=out_dtype, device=x.device)
-        f = _none(x, torch.float32)
-        p = post if a is not None else (f, f, f)
-        _seq().dyt_residual(out, x, a if a is not None else _none(x, out_dtype), *p, *nxt)
+        _seq().dyt_residual(out, x, a, *post, *nxt)
         return out
     return torch_ref.dyt_residual(x, a, post, nxt, out_dtype)
+
+
+def embed_dyt(ids, table, scale: float, nxt):
+    """The stream's start: (x, h) with x = table[ids] * scale in fp32 and h =
+    tanh(alpha x) w + b with nxt in the table's dtype."""
+    if _gpu(table):
+        x = torch.empty((ids.numel(), table.shape[1]), dtype=torch.float32, device=table.device)
+        h = torch.empty(x.shape, dtype=table.dtype, device=table.device)
+        _seq().embed_dyt(h, x, ids, table, float(scale), *nxt)
+        return x, h
+    return torch_ref.embed_dyt(ids, table, scale, nxt)
 
 
 def rmsnorm_rows(x, weight, eps):

@@ -91,7 +91,7 @@ void seq_launch_gated_delta_rule(float*, const void*, const void*, const void*, 
                                  const int*, const int*, const int*, int, int, int, int, int, int, int, int, int,
                                  int, int, int, hipStream_t);
 void seq_launch_dyt_residual(void*, float*, const void*, const float*, const float*, const float*, const float*,
-                             const float*, const float*, int, int, int, hipStream_t);
+                             const float*, const float*, const int64_t*, const void*, float, int, int, int, hipStream_t);
 void seq_launch_rmsnorm_rows(void*, const void*, const float*, int, int, int, float, int, hipStream_t);
 void seq_launch_conv_qkv_store(void*, const void*, const float*, void*, const int*, const int*, const int*,
                                const int*, const int64_t*, void*, void*, const int64_t*, int, int, int, int, int, int,
@@ -1028,24 +1028,33 @@ void ssd_recurrence(torch::Tensor o, torch::Tensor x, torch::Tensor Bm, torch::T
 
 // ---- dynamic-tanh norms, differential attention ----------------------------------
 
-// a / alpha_p / w_p / b_p empty: the stream stays as it is
 void dyt_residual(torch::Tensor out, torch::Tensor x, torch::Tensor a, torch::Tensor alpha_p, torch::Tensor w_p,
                   torch::Tensor b_p, torch::Tensor alpha_n, torch::Tensor w_n, torch::Tensor b_n) {
   CHECK_ACT(out); CHECK_F32C(x); CHECK_F32C(alpha_n); CHECK_F32C(w_n); CHECK_F32C(b_n);
   TORCH_CHECK(x.dim() == 2 && out.is_contiguous() && out.sizes() == x.sizes());
   const int T = x.size(0), W = x.size(1);
   TORCH_CHECK(alpha_n.numel() == 1 && w_n.numel() == W && b_n.numel() == W);
-  const bool has = a.numel() > 0;
-  if (has) {
-    CHECK_ACT(a); CHECK_SAME(a, out); CHECK_F32C(alpha_p); CHECK_F32C(w_p); CHECK_F32C(b_p);
-    TORCH_CHECK(a.is_contiguous() && a.sizes() == x.sizes());
-    TORCH_CHECK(alpha_p.numel() == 1 && w_p.numel() == W && b_p.numel() == W);
-  }
+  CHECK_ACT(a); CHECK_SAME(a, out); CHECK_F32C(alpha_p); CHECK_F32C(w_p); CHECK_F32C(b_p);
+  TORCH_CHECK(a.is_contiguous() && a.sizes() == x.sizes());
+  TORCH_CHECK(alpha_p.numel() == 1 && w_p.numel() == W && b_p.numel() == W);
   if (x.numel() == 0) return;
-  seq_launch_dyt_residual(out.data_ptr(), x.data_ptr<float>(), has ? a.data_ptr() : nullptr,
-                          has ? alpha_p.data_ptr<float>() : nullptr, has ? w_p.data_ptr<float>() : nullptr,
-                          has ? b_p.data_ptr<float>() : nullptr, alpha_n.data_ptr<float>(), w_n.data_ptr<float>(),
-                          b_n.data_ptr<float>(), T, W, f32flag(out), cur_stream());
+  seq_launch_dyt_residual(out.data_ptr(), x.data_ptr<float>(), a.data_ptr(), alpha_p.data_ptr<float>(),
+                          w_p.data_ptr<float>(), b_p.data_ptr<float>(), alpha_n.data_ptr<float>(), w_n.data_ptr<float>(),
+                          b_n.data_ptr<float>(), nullptr, nullptr, 1.0f, T, W, f32flag(out), cur_stream());
+}
+
+// x = table[ids] * scale (fp32), out = tanh(alpha x) w + b
+void embed_dyt(torch::Tensor out, torch::Tensor x, torch::Tensor ids, torch::Tensor table, double scale,
+               torch::Tensor alpha, torch::Tensor w, torch::Tensor b) {
+  CHECK_ACT(out); CHECK_F32C(x); CHECK_I64C(ids); CHECK_ACT(table); CHECK_SAME(table, out); CHECK_F32C(alpha);
+  CHECK_F32C(w); CHECK_F32C(b);
+  TORCH_CHECK(table.is_contiguous() && table.dim() == 2 && x.dim() == 2 && out.is_contiguous() && out.sizes() == x.sizes());
+  const int T = x.size(0), W = x.size(1);
+  TORCH_CHECK(ids.numel() == T && table.size(1) == W && alpha.numel() == 1 && w.numel() == W && b.numel() == W);
+  if (x.numel() == 0) return;
+  seq_launch_dyt_residual(out.data_ptr(), x.data_ptr<float>(), nullptr, nullptr, nullptr, nullptr,
+                          alpha.data_ptr<float>(), w.data_ptr<float>(), b.data_ptr<float>(), ids.data_ptr<int64_t>(),
+                          table.data_ptr(), (float)scale, T, W, f32flag(out), cur_stream());
 }
 
 void rmsnorm_rows(torch::Tensor out, torch::Tensor x, torch::Tensor w, double eps) {
@@ -1200,6 +1209,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("pool_kv_update", &pool_kv_update);
   m.def("ssd_recurrence", &ssd_recurrence);
   m.def("dyt_residual", &dyt_residual);
+  m.def("embed_dyt", &embed_dyt);
   m.def("rmsnorm_rows", &rmsnorm_rows);
   m.def("conv_qkv_store", &conv_qkv_store);
   m.def("attn_diff_mfma_fits", &attn_diff_mfma_fits);

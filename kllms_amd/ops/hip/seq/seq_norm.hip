@@ -389,14 +389,16 @@ __global__ void scale_softcap_kernel(float* __restrict__ z, int64_t n, float sca
 }
 
 // ---- dynamic-tanh norm: tanh(alpha v) w + b, no statistics -------------------------
-// x (fp32 stream) += tanh(alpha_p a) w_p + b_p (a == nullptr: x as it is), then
-// out = tanh(alpha_n x) w_n + b_n. A thread keeps VEC columns of both norms in
+// x (fp32 stream) += tanh(alpha_p a) w_p + b_p, then
+// out = tanh(alpha_n x) w_n + b_n. With ids (and no a) the stream starts here:
+// x = table row of the token times emb_scale. A thread keeps VEC columns of both norms in
 // registers and walks the rows blockIdx.y, + gridDim.y, ...
 template <typename T, int VEC>
 __global__ void __launch_bounds__(256) dyt_residual_kernel(
     T* __restrict__ out, float* __restrict__ x, const T* __restrict__ a, const float* __restrict__ alpha_p,
     const float* __restrict__ w_p, const float* __restrict__ b_p, const float* __restrict__ alpha_n,
-    const float* __restrict__ w_n, const float* __restrict__ b_n, int T_, int W) {
+    const float* __restrict__ w_n, const float* __restrict__ b_n, const int64_t* __restrict__ ids,
+    const T* __restrict__ table, float emb_scale, int T_, int W) {
   const int c = (blockIdx.x * blockDim.x + threadIdx.x) * VEC;
   if (c >= W) return;
   float wp[VEC], bp[VEC], wn[VEC], bn[VEC];
@@ -410,7 +412,13 @@ __global__ void __launch_bounds__(256) dyt_residual_kernel(
   }
   for (int64_t t = blockIdx.y; t < T_; t += gridDim.y) {
     float xv[VEC], av[VEC];
-    if constexpr (VEC == 8) {
+    if (ids != nullptr) {
+      const T* row = table + ids[t] * W + c;
+      if constexpr (VEC == 8) ld8(row, xv); else xv[0] = ldf(row);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) xv[e] *= emb_scale;
+      if constexpr (VEC == 8) st8(x + t * W + c, xv); else x[t * W + c] = xv[0];
+    } else if constexpr (VEC == 8) {
       ld8(x + t * W + c, xv);
       if (a != nullptr) ld8(a + t * W + c, av);
     } else {
@@ -581,8 +589,10 @@ extern "C" void seq_launch_gated_act(void* out, const void* gate, const void* up
 
 extern "C" void seq_launch_dyt_residual(void* out, float* x, const void* a, const float* alpha_p, const float* w_p,
                                         const float* b_p, const float* alpha_n, const float* w_n, const float* b_n,
-                                        int T_, int W, int is_f32, hipStream_t st) {
+                                        const int64_t* ids, const void* table, float emb_scale, int T_, int W,
+                                        int is_f32, hipStream_t st) {
   const bool v8 = W % 8 == 0 && aligned16(out) && aligned16(x) && aligned16(w_n) && aligned16(b_n) &&
+                  (ids == nullptr || aligned16(table)) &&
                   (a == nullptr || (aligned16(a) && aligned16(w_p) && aligned16(b_p)));
   const int cols = v8 ? W / 8 : W;
   const int threads = cols >= 256 ? 256 : (cols + WAVE - 1) / WAVE * WAVE;
@@ -592,9 +602,11 @@ extern "C" void seq_launch_dyt_residual(void* out, float* x, const void* a, cons
   if (gy > 65535) gy = 65535;
   DISPATCH_T(is_f32,
              if (v8) hipLaunchKernelGGL((dyt_residual_kernel<T, 8>), dim3(gx, gy), dim3(threads), 0, st, (T*)out, x,
-                                        (const T*)a, alpha_p, w_p, b_p, alpha_n, w_n, b_n, T_, W);
+                                        (const T*)a, alpha_p, w_p, b_p, alpha_n, w_n, b_n, ids, (const T*)table,
+                                        emb_scale, T_, W);
              else hipLaunchKernelGGL((dyt_residual_kernel<T, 1>), dim3(gx, gy), dim3(threads), 0, st, (T*)out, x,
-                                     (const T*)a, alpha_p, w_p, b_p, alpha_n, w_n, b_n, T_, W);)
+                                     (const T*)a, alpha_p, w_p, b_p, alpha_n, w_n, b_n, ids, (const T*)table,
+                                     emb_scale, T_, W);)
 }
 
 extern "C" void seq_launch_rmsnorm_rows(void* out, const void* x, const float* w, int T_, int C, int x_stride,

@@ -1067,11 +1067,16 @@ def _dyt(v, alpha, w, b) -> torch.Tensor:
 
 
 def dyt_residual(x, a, post, nxt, out_dtype) -> torch.Tensor:
-    """x (fp32, in place) += tanh(alpha a) w + b with post = (alpha, w, b), or
-    x as it is when a is None; returns tanh(alpha x) w + b with nxt, cast."""
-    if a is not None:
-        x.add_(_dyt(a.float(), *post))
+    """x (fp32, in place) += tanh(alpha a) w + b with post = (alpha, w, b);
+    returns tanh(alpha x) w + b with nxt, cast."""
+    x.add_(_dyt(a.float(), *post))
     return _dyt(x, *nxt).to(out_dtype)
+
+
+def embed_dyt(ids, table, scale, nxt):
+    """(table[ids] * scale in fp32, its dynamic tanh in the table's dtype)."""
+    x = table[ids].float() * scale
+    return x, _dyt(x, *nxt).to(table.dtype)
 
 
 def rmsnorm_rows(x, weight, eps) -> torch.Tensor:

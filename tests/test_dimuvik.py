@@ -143,7 +143,9 @@ def test_dynamic_tanh():
     want = x + O.dyt(w, "post", a)
     check(xs, want, atol=1e-5)
     check(h, O.dyt(w, "next", want), atol=1e-5)
-    check(ops.dyt_residual(x.float(), None, None, mods["next"].args, torch.float32), O.dyt(w, "next", x), atol=1e-5)
+    x0, h0 = ops.embed_dyt(torch.tensor([3, 0, 3]), x.float(), 1.7, mods["next"].args)
+    check(x0, x[[3, 0, 3]] * 1.7, atol=1e-5)
+    check(h0, O.dyt(w, "next", x[[3, 0, 3]] * 1.7), atol=1e-5)
 
 
 @pytest.mark.parametrize("cuts", CUTS)

@@ -41,9 +41,10 @@ def test_dyt_residual(dtype, T, W):
     x1, x2 = x.clone(), x.clone()
     close(ops.dyt_residual(x1, a, post, nxt, dtype), torch_ref.dyt_residual(x2, a, post, nxt, dtype), dtype)
     torch.testing.assert_close(x1, x2, rtol=1e-6, atol=2e-6)                # the stream is fp32 in both modes
-    x3 = x.clone()
-    close(ops.dyt_residual(x3, None, None, nxt, dtype), torch_ref.dyt_residual(x2.copy_(x), None, None, nxt, dtype), dtype)
-    assert torch.equal(x3, x)
+    table, ids = rnd(50, W, dtype=dtype, seed=6), torch.randint(0, 50, (T,), generator=torch.Generator().manual_seed(7)).to(DEV)
+    (x3, h3), (x4, h4) = ops.embed_dyt(ids, table, 1.7, nxt), torch_ref.embed_dyt(ids, table, 1.7, nxt)
+    torch.testing.assert_close(x3, x4, rtol=1e-6, atol=1e-6)
+    close(h3, h4, dtype)
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
