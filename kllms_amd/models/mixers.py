@@ -679,12 +679,10 @@ class DiffAttention(nn.Module):
         parts = [("q", spec.heads * 2 * spec.dim)]
         if self.own_kv:
             parts += [("k", spec.kv_heads * 2 * spec.dim), ("v", spec.kv_heads * spec.vdim)]
-        self.inp = FusedInput(hidden, parts, dtype)
-        # bias and taps (taps-major) over the fused projection's columns as laid out (zeros in alignment gaps);
-        # both are applied by the convolution kernel
-        C = self.inp.weight.shape[0]
-        self.bias = nn.Parameter(torch.zeros(C, dtype=torch.float32), requires_grad=False)
-        self.conv = nn.Parameter(torch.zeros(spec.conv, C, dtype=torch.float32), requires_grad=False)
+        self.inp = FusedInput(hidden, parts, dtype, bias_parts=[n for n, _ in parts])
+        # taps-major over the fused projection's columns as laid out (zero taps in alignment gaps)
+        self.conv = nn.Parameter(torch.zeros(spec.conv, self.inp.weight.shape[0], dtype=torch.float32),
+                                 requires_grad=False)
         self.lambdas = _param(4, spec.dim, dtype=torch.float32)
         self.lam = 0.0
         self.o_proj = _param(hidden, spec.heads * spec.vdim, dtype=dtype)
@@ -717,8 +715,8 @@ class DiffAttention(nn.Module):
         sp = self.spec
         T = h.shape[0]
         p = self.inp.parts
-        q = ops.conv_qkv_store(self.inp(h), self.conv, self.bias, st.conv, batch.state_slots, batch.cu_seqlens,
-                               batch.seg_start, batch.token_seg, p["q"], sp.temp_coef, sp.temp_every, p.get("k"),
+        q = ops.conv_qkv_store(self.inp(h), self.conv, st.conv, batch.state_slots, batch.cu_seqlens, batch.seg_start,
+                               batch.token_seg, batch.positions, p["q"], sp.temp_coef, sp.temp_every, p.get("k"),
                                p.get("v"), st.k, st.v, batch.slot_mapping, single_rows(batch))
         att = ops.attn_diff_paged(q.view(T, sp.heads, 2 * sp.dim), st.k, st.v, batch.block_tables, batch.token_seg,
                                   batch.positions, sp.scale, self.lam, 1.0 - sp.diff, self.eps, self._tiles(batch))
@@ -727,7 +725,7 @@ class DiffAttention(nn.Module):
     def checkpoint_map(self, pre: str) -> Dict[str, torch.Tensor]:
         m = {}
         for n, (off, size) in self.inp.parts.items():
-            m[pre + n], m[pre + n + ".b"] = self.inp.slot(n), self.bias[off:off + size]
+            m[pre + n], m[pre + n + ".b"] = self.inp.slot(n), self.inp.bias_slot(n)
             m[pre + n + ".conv"] = self.conv.t()[off:off + size]
         for i, n in enumerate(self.LAMBDAS):
             m[pre + n] = self.lambdas[i]

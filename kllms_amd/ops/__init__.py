@@ -893,9 +893,9 @@ def rmsnorm_rows(x, weight, eps):
     return torch_ref.rmsnorm_rows(x, weight, eps)
 
 
-def conv_qkv_store(y, w, bias, conv_state, state_slots, cu_seqlens, seg_start, token_seg, q_cols, temp_coef,
+def conv_qkv_store(y, w, conv_state, state_slots, cu_seqlens, seg_start, token_seg, positions, q_cols, temp_coef,
                    temp_every, k_cols=None, v_cols=None, k_cache=None, v_cache=None, slot_mapping=None, single=False):
-    """Bias [C] fp32 and short causal convolution of a fused projection's rows; k and v columns
+    """Short causal convolution of a fused projection's rows; k and v columns
     into the paged caches, the q columns times the query temperature returned
     packed [T, width]. ``single``: every segment is one row (the history is
     updated by the same launch)."""
@@ -904,12 +904,12 @@ def conv_qkv_store(y, w, bias, conv_state, state_slots, cu_seqlens, seg_start, t
         has = k_cols is not None
         e = _none(y)
         ko, vo = (k_cols[0], v_cols[0]) if has else (0, 0)
-        _seq().conv_qkv_store(q, y, w, bias, conv_state, state_slots, cu_seqlens, seg_start, token_seg,
+        _seq().conv_qkv_store(q, y, w, conv_state, state_slots, cu_seqlens, seg_start, token_seg, positions,
                               int(q_cols[0]), float(temp_coef), int(temp_every), int(ko), int(vo),
                               k_cache if has else e, v_cache if has else e,
                               slot_mapping if has else _none(y, torch.long), bool(single))
         return q
-    return torch_ref.conv_qkv_store(y, w, bias, conv_state, state_slots, cu_seqlens, seg_start, q_cols, temp_coef,
+    return torch_ref.conv_qkv_store(y, w, conv_state, state_slots, cu_seqlens, seg_start, positions, q_cols, temp_coef,
                                     temp_every, k_cols, v_cols, k_cache, v_cache, slot_mapping)
 
 

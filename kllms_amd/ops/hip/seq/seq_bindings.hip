@@ -93,8 +93,8 @@ void seq_launch_gated_delta_rule(float*, const void*, const void*, const void*, 
 void seq_launch_dyt_residual(void*, float*, const void*, const float*, const float*, const float*, const float*,
                              const float*, const float*, const int64_t*, const void*, float, int, int, int, hipStream_t);
 void seq_launch_rmsnorm_rows(void*, const void*, const float*, int, int, int, float, int, hipStream_t);
-void seq_launch_conv_qkv_store(void*, const void*, const float*, const float*, void*, const int*, const int*,
-                               const int*, const int*, void*, void*, const int64_t*, int, int, int, int, int, int,
+void seq_launch_conv_qkv_store(void*, const void*, const float*, void*, const int*, const int*, const int*,
+                               const int*, const int64_t*, void*, void*, const int64_t*, int, int, int, int, int, int,
                                int, int, int, int, int, int, int, int, int, float, int, int, int, hipStream_t);
 int seq_diff_mfma_fits(int, int);
 int seq_launch_attn_diff_paged(void*, const void*, const void*, const void*, const int*, const int*, const int64_t*,
@@ -1065,24 +1065,23 @@ void rmsnorm_rows(torch::Tensor out, torch::Tensor x, torch::Tensor w, double ep
                           (int)x.stride(0), (float)eps, f32flag(out), cur_stream());
 }
 
-// y [T, C] rows of a fused projection, bias [C] added on the way in; q_out [T, width] = columns qo..; caches [NB, G, BS, D | V] take the
+// y [T, C] rows of a fused projection; q_out [T, width] = columns qo..; caches [NB, G, BS, D | V] take the
 // columns from ko and vo (caches empty: q only). single: every segment is one row
-void conv_qkv_store(torch::Tensor q_out, torch::Tensor y, torch::Tensor w, torch::Tensor bias, torch::Tensor hist,
-                    torch::Tensor slots, torch::Tensor cu, torch::Tensor seg_start, torch::Tensor token_seg, int64_t qo,
-                    double coef, int64_t every, int64_t ko, int64_t vo, torch::Tensor k_cache,
+void conv_qkv_store(torch::Tensor q_out, torch::Tensor y, torch::Tensor w, torch::Tensor hist, torch::Tensor slots,
+                    torch::Tensor cu, torch::Tensor seg_start, torch::Tensor token_seg, torch::Tensor positions,
+                    int64_t qo, double coef, int64_t every, int64_t ko, int64_t vo, torch::Tensor k_cache,
                     torch::Tensor v_cache, torch::Tensor slot_map, bool single) {
-  CHECK_ACT(y); CHECK_ROWS2(y); CHECK_SAME(q_out, y); CHECK_SAME(hist, y); CHECK_F32C(w); CHECK_F32C(bias);
-  CHECK_I32C(token_seg);
+  CHECK_ACT(y); CHECK_ROWS2(y); CHECK_SAME(q_out, y); CHECK_SAME(hist, y); CHECK_F32C(w); CHECK_I32C(token_seg);
+  CHECK_I64C(positions);
   check_segments(slots, cu, seg_start, hist);
   const int T = y.size(0), C = y.size(1), B = slots.numel();
   TORCH_CHECK(w.dim() == 2 && w.size(1) == C && w.size(0) >= 1 && w.size(0) <= 16, "1..16 convolution taps supported");
   const int K = w.size(0);
-  TORCH_CHECK(bias.numel() == C);
   TORCH_CHECK(hist.dim() == 3 && hist.size(1) == K - 1 && hist.size(2) == C);
   TORCH_CHECK(q_out.is_cuda() && q_out.is_contiguous() && q_out.dim() == 2 && q_out.size(0) == T);
   const int64_t qn = q_out.size(1);
   TORCH_CHECK(qo >= 0 && qo + qn <= C && every >= 1 && every < (1LL << 31));
-  TORCH_CHECK(token_seg.numel() == T && (!single || B == T));
+  TORCH_CHECK(token_seg.numel() == T && positions.numel() == T && (!single || B == T));
   int64_t kn = 0, vn = 0;
   int G = 1, D2 = 1, V = 1, BS = 1;
   const bool has = k_cache.numel() > 0;
@@ -1098,9 +1097,9 @@ void conv_qkv_store(torch::Tensor q_out, torch::Tensor y, torch::Tensor w, torch
                 "column ranges overlap");
   }
   if (T == 0 || B == 0) return;
-  seq_launch_conv_qkv_store(q_out.data_ptr(), y.data_ptr(), w.data_ptr<float>(), bias.data_ptr<float>(),
-                            hist.data_ptr(), slots.data_ptr<int>(), cu.data_ptr<int>(), seg_start.data_ptr<int>(),
-                            token_seg.data_ptr<int>(), has ? k_cache.data_ptr() : nullptr,
+  seq_launch_conv_qkv_store(q_out.data_ptr(), y.data_ptr(), w.data_ptr<float>(), hist.data_ptr(), slots.data_ptr<int>(),
+                            cu.data_ptr<int>(), seg_start.data_ptr<int>(), token_seg.data_ptr<int>(),
+                            positions.data_ptr<int64_t>(), has ? k_cache.data_ptr() : nullptr,
                             has ? v_cache.data_ptr() : nullptr, has ? slot_map.data_ptr<int64_t>() : nullptr, T, B, C, K,
                             (int)y.stride(0), (int)qo, (int)qn, (int)ko, (int)kn, (int)vo, (int)vn, D2, V, G, BS,
                             (float)coef, (int)every, single ? 1 : 0, f32flag(y), cur_stream());

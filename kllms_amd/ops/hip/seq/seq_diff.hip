@@ -1,8 +1,8 @@
 // Differential attention: every head holds two softmax maps over the same
 // values, combined as a_1 - lambda a_2 and RMS-normed per head. Queries, keys
 // and values pass a short causal convolution on the way in. The kernels:
-//   conv_qkv_store   bias and convolution of a fused q | k | v projection, k and v
-//                    into the paged caches, q times the query temperature (one launch)
+//   conv_qkv_store   convolution of a fused q | k | v projection, k and v into
+//                    the paged caches, q times the query temperature (one launch)
 //   attn_diff_paged  both maps, the combination and the norm over the paged
 //                    cache, plain causal
 //     - a plain kernel (any size, bf16 or fp32; the exact-mode path)
@@ -26,22 +26,19 @@ __device__ __forceinline__ void stv(T* p, const float v[VEC]) {
   if constexpr (VEC == 8) st8(p, v); else stf(p, v[0]);
 }
 
-// ---- step input: bias, short convolution, query temperature, paged store -----------
-// z_t = sum_j w[j] (y_{t-K+1+j} + bias), where rows before the sequence's start are
-// zero and carry no bias. A thread owns VEC columns of `run` consecutive rows. KT > 0: up to KT taps with
+// ---- step input: short convolution, query temperature, paged store -----------------
+// A thread owns VEC columns of `run` consecutive rows. KT > 0: up to KT taps with
 // the taps and the last KT rows in registers (missing leading taps are zero);
 // KT == 0: any number of taps, rows re-read. Rows before a segment come from
-// hist [slot, K-1, C] (oldest first, without the bias), zeros for a fresh
-// sequence. Columns
+// hist [slot, K-1, C] (oldest first), zeros for a fresh sequence. Columns
 // [qo, qo + qn) go to q_out times 1 + coef ln(floor((p + 1) / every) + 1);
 // [ko, ko + kn) and [vo, vo + vn) to the caches; the rest are alignment gaps.
 // single: every segment is one row, and the thread moves its columns' history on.
 template <typename T, int VEC, int KT>
 __global__ void __launch_bounds__(256) conv_qkv_store_kernel(
-    T* __restrict__ q_out, const T* __restrict__ y, const float* __restrict__ w, const float* __restrict__ bias,
-    T* __restrict__ hist_,
+    T* __restrict__ q_out, const T* __restrict__ y, const float* __restrict__ w, T* __restrict__ hist_,
     const int* __restrict__ slots, const int* __restrict__ cu, const int* __restrict__ seg_start,
-    const int* __restrict__ token_seg, T* __restrict__ kc, T* __restrict__ vc,
+    const int* __restrict__ token_seg, const int64_t* __restrict__ positions, T* __restrict__ kc, T* __restrict__ vc,
     const int64_t* __restrict__ slot_map, int T_, int C, int K, int y_stride, int qo, int qn, int ko, int kn, int vo,
     int vn, int D2, int V, int G, int BS, float coef, int every, int run, int single) {
   const int c = (blockIdx.x * blockDim.x + threadIdx.x) * VEC;
@@ -53,8 +50,7 @@ __global__ void __launch_bounds__(256) conv_qkv_store_kernel(
   const int cc = isk ? c - ko : c - vo;
   const int g = (isk || isv) ? cc / hw : 0, ce = cc - g * hw;
   constexpr int KW = KT > 0 ? KT : 1;
-  float wt[KW][VEC], win[KW][VEC], bv[VEC];
-  ldv<VEC>(bias + c, bv);
+  float wt[KW][VEC], win[KW][VEC];
   if (KT > 0) {
 #pragma unroll
     for (int j = 0; j < KW; ++j) {
@@ -68,7 +64,6 @@ __global__ void __launch_bounds__(256) conv_qkv_store_kernel(
   for (int t = t0; t < t1; ++t) {
     const int b = token_seg[t];
     const int i = t - cu[b];
-    const int p = seg_start[b] + i;                   // position in the sequence: p + 1 rows exist up to here
     const bool fresh = seg_start[b] == 0;
     T* hist = hist_ + (int64_t)slots[b] * (K - 1) * C + c;
     float acc[VEC];
@@ -96,7 +91,7 @@ __global__ void __launch_bounds__(256) conv_qkv_store_kernel(
 #pragma unroll
       for (int j = 0; j < KW; ++j)
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) acc[e] += wt[j][e] * (KW - 1 - j <= p ? win[j][e] + bv[e] : 0.f);
+        for (int e = 0; e < VEC; ++e) acc[e] += wt[j][e] * win[j][e];
       if (single) {
 #pragma unroll
         for (int j = 1; j < KW; ++j)
@@ -107,13 +102,13 @@ __global__ void __launch_bounds__(256) conv_qkv_store_kernel(
       for (int e = 0; e < VEC; ++e) acc[e] = 0.f;
       for (int j = 0; j < K; ++j) {
         const int src = i - (K - 1 - j);
-        if (p - (K - 1 - j) < 0) continue;             // before the sequence's start
         float xv[VEC], wv[VEC];
         if (src >= 0) ldv<VEC>(y + (int64_t)(t - (K - 1 - j)) * y_stride + c, xv);
-        else ldv<VEC>(hist + (int64_t)(K - 1 + src) * C, xv);
+        else if (!fresh) ldv<VEC>(hist + (int64_t)(K - 1 + src) * C, xv);
+        else continue;
         ldv<VEC>(w + (int64_t)j * C + c, wv);
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) acc[e] += wv[e] * (xv[e] + bv[e]);
+        for (int e = 0; e < VEC; ++e) acc[e] += wv[e] * xv[e];
       }
       if (single) {                                   // oldest first: every row is read before it is overwritten
         float xv[VEC];
@@ -130,7 +125,7 @@ __global__ void __launch_bounds__(256) conv_qkv_store_kernel(
     }
     if (isq) {
       if (coef != 0.f) {
-        const float temp = 1.0f + coef * logf((float)((p + 1) / every + 1));
+        const float temp = 1.0f + coef * logf((float)((positions[t] + 1) / every + 1));
 #pragma unroll
         for (int e = 0; e < VEC; ++e) acc[e] *= temp;
       }
@@ -623,14 +618,14 @@ __global__ void __launch_bounds__(256) attn_diff_merge_kernel(
 extern "C" void seq_launch_conv_state_update(const void*, void*, const int*, const int*, const int*, int, int, int,
                                              int, int, hipStream_t);
 
-extern "C" void seq_launch_conv_qkv_store(void* q_out, const void* y, const float* w, const float* bias, void* hist,
-                                          const int* slots, const int* cu, const int* seg_start,
-                                          const int* token_seg, void* kc, void* vc, const int64_t* slot_map,
+extern "C" void seq_launch_conv_qkv_store(void* q_out, const void* y, const float* w, void* hist, const int* slots,
+                                          const int* cu, const int* seg_start, const int* token_seg,
+                                          const int64_t* positions, void* kc, void* vc, const int64_t* slot_map,
                                           int T_, int B, int C, int K, int y_stride, int qo, int qn, int ko, int kn,
                                           int vo, int vn, int D2, int V, int G, int BS, float coef, int every,
                                           int single, int is_f32, hipStream_t st) {
   bool v8 = C % 8 == 0 && y_stride % 8 == 0 && qo % 8 == 0 && qn % 8 == 0 && aligned16(q_out) && aligned16(y) &&
-            aligned16(w) && aligned16(bias) && aligned16(hist);
+            aligned16(w) && aligned16(hist);
   if (kn > 0) v8 = v8 && ko % 8 == 0 && vo % 8 == 0 && D2 % 8 == 0 && V % 8 == 0 && aligned16(kc) && aligned16(vc);
   const int gx = (C / (v8 ? 8 : 1) + 255) / 256;
   // rows per thread: long enough to reuse the window, short enough to fill the chip
@@ -640,7 +635,7 @@ extern "C" void seq_launch_conv_qkv_store(void* q_out, const void* y, const floa
   const dim3 grid(gx, (T_ + run - 1) / run);
 #define CONV_LAUNCH(VEC, KT)                                                                                       \
   DISPATCH_T(is_f32, hipLaunchKernelGGL((conv_qkv_store_kernel<T, VEC, KT>), grid, dim3(256), 0, st, (T*)q_out,    \
-                                        (const T*)y, w, bias, (T*)hist, slots, cu, seg_start, token_seg,           \
+                                        (const T*)y, w, (T*)hist, slots, cu, seg_start, token_seg, positions,      \
                                         (T*)kc, (T*)vc, slot_map, T_, C, K, y_stride, qo, qn, ko, kn, vo, vn, D2,  \
                                         V, G, BS, coef, every, run, single);)
   if (v8 && K <= 4) { CONV_LAUNCH(8, 4) }

@@ -1084,13 +1084,12 @@ def rmsnorm_rows(x, weight, eps) -> torch.Tensor:
     return rmsnorm_cast(x, weight, eps, x.dtype)
 
 
-def conv_qkv_store(y, w, bias, conv_state, state_slots, cu_seqlens, seg_start, q_cols, temp_coef, temp_every,
+def conv_qkv_store(y, w, conv_state, state_slots, cu_seqlens, seg_start, positions, q_cols, temp_coef, temp_every,
                    k_cols, v_cols, k_cache, v_cache, slot_mapping) -> torch.Tensor:
     """Per-channel causal convolution over time of a projection's rows
-    y [T, C] + bias [C] (w [K, C] taps-major, last row = current token;
-    conv_state [slots, K-1, C] holds the last K-1 rows without the bias and is
-    updated), without an activation; rows before the sequence's start are zero
-    and have no bias. (offset, width) column ranges: the k and v columns go to the
+    y [T, C] (w [K, C] taps-major, last row = current token; conv_state
+    [slots, K-1, C] holds the last K-1 rows and is updated), without an
+    activation. (offset, width) column ranges: the k and v columns go to the
     paged caches [NB, G, BS, D | Dv] at the flat slots, the q columns times
     1 + temp_coef ln(floor((p + 1) / temp_every) + 1) are returned."""
     T, C = y.shape
@@ -1098,17 +1097,13 @@ def conv_qkv_store(y, w, bias, conv_state, state_slots, cu_seqlens, seg_start, q
     z = torch.empty(T, C, dtype=torch.float32, device=y.device)
     cu, st, sl = cu_seqlens.tolist(), seg_start.tolist(), state_slots.tolist()
     wf = w.float()
-    pos = torch.zeros(T, dtype=torch.long, device=y.device)
     for b in range(len(sl)):
         s, e = cu[b], cu[b + 1]
         if e == s:
             continue
         hist = conv_state[sl[b]].float() if st[b] > 0 else torch.zeros(K - 1, C, device=y.device)
         ext = torch.cat([hist, y[s:e].float()], 0)
-        there = torch.arange(st[b] - (K - 1), st[b] + e - s, device=y.device) >= 0
-        full = torch.where(there[:, None], ext + bias.float(), torch.zeros_like(ext))
-        z[s:e] = sum(full[j:j + (e - s)] * wf[j] for j in range(K))
-        pos[s:e] = torch.arange(st[b], st[b] + e - s, device=y.device)
+        z[s:e] = sum(ext[j:j + (e - s)] * wf[j] for j in range(K))
         if K > 1:
             conv_state[sl[b]] = ext[ext.shape[0] - (K - 1):].to(conv_state.dtype)
     if k_cols is not None:
@@ -1116,7 +1111,7 @@ def conv_qkv_store(y, w, bias, conv_state, state_slots, cu_seqlens, seg_start, q
         blk, off = slot_mapping // BS, slot_mapping % BS
         for (o, n), cache in ((k_cols, k_cache), (v_cols, v_cache)):
             cache[blk, :, off] = z[:, o:o + n].view(T, G, -1).to(cache.dtype)
-    temp = 1.0 + temp_coef * torch.log(((pos + 1) // temp_every + 1).float())
+    temp = 1.0 + temp_coef * torch.log(((positions + 1) // temp_every + 1).float())
     return (z[:, q_cols[0]:q_cols[0] + q_cols[1]] * temp[:, None]).to(y.dtype)
 
 

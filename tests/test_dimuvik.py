@@ -158,10 +158,9 @@ def test_diff_attention(cuts, heads, kv_heads, dim, vdim, conv):
 
 
 def test_short_convolution_across_portions_and_the_start():
-    """Rows before the sequence count as zero whatever the slot held, without
-    the bias, which every row of the sequence gets before the convolution."""
-    taps, raw, bias = rows(5, 3, 6), rows(7, 5, 7), 2.0 + rows(1, 5, 5)[0]
-    u = raw + bias
+    """Rows before the sequence count as zero whatever the slot held; biases
+    enter the carried rows (they are added before the convolution)."""
+    taps, u = rows(5, 3, 6), rows(7, 5, 7)
     y = O.short_conv(u, taps)
     check(y[0], taps[:, 2] * u[0], atol=1e-12)
     check(y[4], taps[:, 0] * u[2] + taps[:, 1] * u[3] + taps[:, 2] * u[4], atol=1e-12)
@@ -169,10 +168,10 @@ def test_short_convolution_across_portions_and_the_start():
     hist = torch.full((2, 2, 5), 9.0)
     got = []
     for start, n in [(0, 1), (1, 1), (2, 3), (5, 2)]:
-        got.append(ops.conv_qkv_store(raw[start:start + n].float(), taps.t().contiguous().float(), bias.float(), hist, i32([1]),
-                                      i32([0, n]), i32([start]), i32([0] * n), (0, 5), 0.0, 1))
+        got.append(ops.conv_qkv_store(u[start:start + n].float(), taps.t().contiguous().float(), hist, i32([1]), i32([0, n]),
+                                      i32([start]), i32([0] * n), torch.arange(start, start + n), (0, 5), 0.0, 1))
     check(torch.cat(got), y, atol=1e-5)
-    assert torch.equal(hist[0], torch.full((2, 5), 9.0)) and torch.equal(hist[1], raw[5:7].float())
+    assert torch.equal(hist[0], torch.full((2, 5), 9.0)) and torch.equal(hist[1], u[5:7].float())
     lay = layer("attention", att(), None)
     w = O.random_weights(model_cfg([lay]), 8)
     w["l0.mix.k.b"] = w["l0.mix.k.b"] + 2.0
@@ -188,8 +187,8 @@ def test_query_temperature_steps_at_its_edges(coef, every):
     assert abs(O.query_temperature(3 * every - 1, coef, every) - (1 + coef * math.log(4))) < 1e-12
     i32 = lambda x: torch.tensor(x, dtype=torch.int32)
     n = 4 * every + 1
-    q = ops.conv_qkv_store(torch.ones(n, 2), torch.ones(1, 2), torch.zeros(2), torch.zeros(1, 0, 2), i32([0]), i32([0, n]), i32([0]),
-                           i32([0] * n), (0, 2), coef, every)
+    q = ops.conv_qkv_store(torch.ones(n, 2), torch.ones(1, 2), torch.zeros(1, 0, 2), i32([0]), i32([0, n]), i32([0]), i32([0] * n),
+                           torch.arange(n), (0, 2), coef, every)
     check(q[:, 0], torch.tensor([O.query_temperature(p, coef, every) for p in range(n)], dtype=torch.float64), atol=1e-6)
     lay = layer("attention", att(coef=coef, every=every, scale=1.0), None)
     w = O.random_weights(model_cfg([lay]), 10)

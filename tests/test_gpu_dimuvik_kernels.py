@@ -87,15 +87,15 @@ def test_conv_qkv_store(dtype, K, H, G, D2, V, BS, own):
         q_cols, k_cols = (0, H * D2), (al(H * D2), G * D2)
         v_cols = (k_cols[0] + al(G * D2), G * V)
         C = v_cols[0] + al(G * V) if own else al(H * D2)
-        y, w, bias = rnd(sum(ln), C, dtype=dtype), rnd(K, C, std=0.5, seed=5), rnd(C, seed=8)
+        y, w = rnd(sum(ln), C, dtype=dtype), rnd(K, C, std=0.5, seed=5)
         hist = rnd(7, K - 1, C, dtype=dtype, seed=6)
         cu = i32([0] + torch.tensor(ln).cumsum(0).tolist())
         slots, seg_start = i32([3, 0, 6, 1, 4]), i32(starts)
         h1, h2 = hist.clone(), hist.clone()
         k1, k2, v1, v2 = c["k"].clone(), c["k"].clone(), c["v"].clone(), c["v"].clone()
         kv = lambda k, v: (k_cols, v_cols, k, v, c["slots"]) if own else (None, None, None, None, None)
-        q1 = ops.conv_qkv_store(y, w, bias, h1, slots, cu, seg_start, c["seg"], q_cols, 0.3, 8, *kv(k1, v1), single)
-        q2 = torch_ref.conv_qkv_store(y, w, bias, h2, slots, cu, seg_start, q_cols, 0.3, 8, *kv(k2, v2))
+        q1 = ops.conv_qkv_store(y, w, h1, slots, cu, seg_start, c["seg"], c["pos"], q_cols, 0.3, 8, *kv(k1, v1), single)
+        q2 = torch_ref.conv_qkv_store(y, w, h2, slots, cu, seg_start, c["pos"], q_cols, 0.3, 8, *kv(k2, v2))
         close(q1, q2, dtype)
         close(k1, k2, dtype)
         close(v1, v2, dtype)
