@@ -1124,7 +1124,7 @@ MODEL_PRESETS: dict = {
         vocab=512, width=64, depth=4, a_heads=4, a_kv=2, a_dim=8, a_vdim=24, heads=4, dim=16, rot_dim=8, vdim=24,
         kv_rank=32, q_rank=24, ff=96, experts=6, top=2, expert_ff=48, shared_ff=40),
     "mid-dimuvik": _dimuvik_preset(
-        vocab=2048, width=512, depth=4, a_heads=4, a_kv=2, a_dim=64, a_vdim=128, heads=8, dim=64, rot_dim=32, vdim=64,
+        vocab=2048, width=512, depth=4, a_heads=4, a_kv=2, a_dim=64, a_vdim=128, heads=4, dim=64, rot_dim=64, vdim=64,
         kv_rank=128, q_rank=192, ff=1024, experts=8, top=2, expert_ff=256, shared_ff=256),
     # layer shapes of real models at reduced depth, beside llama-/mitunex-{1b,8b}-l6
     "dimuvik-8b-l6": _dimuvik_preset(

@@ -94,8 +94,8 @@ def test_conv_qkv_store(dtype, K, H, G, D2, V, BS, own):
         h1, h2 = hist.clone(), hist.clone()
         k1, k2, v1, v2 = c["k"].clone(), c["k"].clone(), c["v"].clone(), c["v"].clone()
         kv = lambda k, v: (k_cols, v_cols, k, v, c["slots"]) if own else (None, None, None, None, None)
-        q1 = ops.conv_qkv_store(y, w, h1, slots, cu, seg_start, c["seg"], c["pos"], q_cols, 0.3, 8, *kv(k1, v1), single)
-        q2 = torch_ref.conv_qkv_store(y, w, h2, slots, cu, seg_start, c["pos"], q_cols, 0.3, 8, *kv(k2, v2))
+        q1 = ops.conv_qkv_store(y, w, h1, slots, cu, seg_start, c["seg"], c["pos"], q_cols, 0.35, 8, *kv(k1, v1), single)
+        q2 = torch_ref.conv_qkv_store(y, w, h2, slots, cu, seg_start, c["pos"], q_cols, 0.35, 8, *kv(k2, v2))
         close(q1, q2, dtype)
         close(k1, k2, dtype)
         close(v1, v2, dtype)
@@ -105,7 +105,7 @@ def test_conv_qkv_store(dtype, K, H, G, D2, V, BS, own):
         assert torch.equal(h1[[2, 5]], hist[[2, 5]])               # slots no segment names stay as they were
 
 
-SIZES = [(4, 2, 8, 24), (3, 3, 48, 96), (4, 1, 64, 64), (8, 2, 128, 256), (6, 2, 40, 72), (5, 1, 16, 8), (2, 1, 128, 32),
+SIZES = [(4, 2, 8, 24), (3, 3, 48, 104), (4, 1, 64, 64), (8, 2, 128, 256), (6, 2, 40, 72), (5, 1, 16, 8), (2, 1, 128, 32),
          (1, 1, 24, 200), (2, 2, 5, 7), (40, 1, 8, 16), (3, 1, 136, 40), (4, 4, 32, 136)]
 
 
@@ -132,7 +132,7 @@ def test_attn_diff_over_segments(dtype, H, G, D, V):
 
 
 @pytest.mark.parametrize("splits", [0, 1, 2, 5, 64])
-@pytest.mark.parametrize("H,G,D,V,BS", [(8, 2, 128, 256, 16), (4, 4, 48, 96, 4), (3, 1, 16, 40, 64)])
+@pytest.mark.parametrize("H,G,D,V,BS", [(8, 2, 128, 256, 16), (4, 4, 40, 88, 4), (3, 1, 16, 40, 64)])
 def test_attn_diff_single_rows_and_key_shares(splits, H, G, D, V, BS):
     """Decode: rows of very different lengths; more shares than a short row has tiles."""
     starts = [0, 1, 63, 64, 65, 700, 333]
@@ -161,11 +161,11 @@ def test_diff_tiles_plan():
     assert tiles.tolist() == [[72, 2], [65, 6], [33, 32], [1, 32]]
 
 
-@pytest.mark.parametrize("T,N,top", [(1, 4, 2), (33, 8, 4), (5, 6, 6)])
+@pytest.mark.parametrize("T,N,top", [(1, 4, 2), (33, 9, 4), (5, 6, 6)])
 def test_route_scale_and_ungated_shared_expert(T, N, top):
     z, corr = rnd(T, N), rnd(N, std=0.3, seed=1)
-    i1, w1 = ops.moe_route(z, corr, top, 1, 1, "softmax", False, 2.5)
-    i2, w2 = torch_ref.moe_route(z, corr, top, 1, 1, "softmax", False, 2.5)
+    i1, w1 = ops.moe_route(z, corr, top, 1, 1, "softmax", False, 1.9)
+    i2, w2 = torch_ref.moe_route(z, corr, top, 1, 1, "softmax", False, 1.9)
     assert torch.equal(i1, i2)
     close(w1, w2, torch.float32)
     for W in (16, 13):
